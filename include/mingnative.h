@@ -28,7 +28,7 @@
 extern "C" {
 #endif
 
-#define MN_VERSION 129 /* 0.1.29: post-norm mixed-mixer sequence models (section 12).  0.1.28: hybrid-mixer sequence models (section 11).  0.1.27: parallel-mixer sequence models (section 10).  0.1.26: latent-cache sequence models (section 9).  0.1.24: mn_persist_set_status_word; mn_tp_allreduce PUSH|REDUCE above the one-shot row limit implies GATHER.  0.1.23: ABI guards mn_sizeof_* / mn_struct_layout.  0.1.20: fp8 weight mode (section 7): wfmt / row-scale fields at the END of mn_skinny_args, mn_rf_head,
+#define MN_VERSION 130 /* 0.1.30: layers with a decay per key channel and mixed attention heads (section 13).  0.1.29: post-norm mixed-mixer sequence models (section 12).  0.1.28: hybrid-mixer sequence models (section 11).  0.1.27: parallel-mixer sequence models (section 10).  0.1.26: latent-cache sequence models (section 9).  0.1.24: mn_persist_set_status_word; mn_tp_allreduce PUSH|REDUCE above the one-shot row limit implies GATHER.  0.1.23: ABI guards mn_sizeof_* / mn_struct_layout.  0.1.20: fp8 weight mode (section 7): wfmt / row-scale fields at the END of mn_skinny_args, mn_rf_head,
                           mn_llm and mn_llm_tp (zero = bf16: callers of 0.1.10 that zero-fill the structs are unchanged),
                           mn_quant_fp8_rows / mn_dequant_fp8_rows / mn_stream_mfma_w8 / mn_stream_mfma_grouped_w8 */
 
@@ -903,6 +903,11 @@ MN_API int mn_rotary_frequencies_host(int dims, double base, double factor, doub
 MN_API int mn_rope_unit_append(const float* qkv, int64_t ldqkv, int M, int H, int G, int dim, int vdim, int rot_dims, const float* freq,
                                float mag, int unit, float eps, float q_scale, const int32_t* row_seq, const int32_t* row_slot, float* q_out,
                                int64_t ldq, float* k_arena, float* v_arena, int t_max, void* stream);
+/* The same with the first value head at column v_col of a row: v_col = H * dim makes the values the keys as they were projected (before
+ * rotation and norm). */
+MN_API int mn_rope_unit_append_from(const float* qkv, int64_t ldqkv, int M, int H, int G, int dim, int vdim, int v_col, int rot_dims,
+                                    const float* freq, float mag, int unit, float eps, float q_scale, const int32_t* row_seq,
+                                    const int32_t* row_slot, float* q_out, int64_t ldq, float* k_arena, float* v_arena, int t_max, void* stream);
 /* Decode rows (every row alone in its sequence) in one launch: qkv holds the UNFILTERED projections; every channel goes through the
  * causal filter w_conv bf16 [channels, conv] over the sequence's earlier inputs in conv_state fp32 [n_seq, conv - 1, channels], which
  * moves on by this row (conv 0: no filter); then mn_rope_unit_append; then, for a row that completes a block of `pool` slots, the
@@ -1104,29 +1109,51 @@ MN_API int mn_moe_combine_pass_residual(float* x, int64_t ldx, const float* y, i
                                         const float* w, int top, int n_real, const float* h, int64_t ldh, const float* add, int64_t ldadd,
                                         int M, int n, void* stream);
 
-enum { MN_HYB_ATTENTION = 0, MN_HYB_LIGHTNING = 1 };
+/* Mixers of the hybrid step function: the two above, and the mixers of section 13 */
+enum { MN_HYB_ATTENTION = 0, MN_HYB_LIGHTNING = 1, MN_HYB_TALK_ATTENTION = 2, MN_HYB_CHANNEL_DELTA = 3, MN_HYB_GLA = 4 };
 enum { MN_HYB_FF_NONE = 0, MN_HYB_FF_DENSE = 1, MN_HYB_FF_MOE = 2 };
+enum { MN_HYB_ACT_RELU2 = 0, MN_HYB_ACT_XIELU = 1 };       /* of the dense / shared feed-forward */
+enum { MN_HYB_NORM_RMS = 0, MN_HYB_NORM_LAYER = 1 };
 typedef struct mn_hyb_layer {
-  int32_t kind;                                    /* MN_HYB_ATTENTION | MN_HYB_LIGHTNING */
-  int32_t heads, kv_heads, dim, vdim;              /* lightning: kv_heads = heads */
+  int32_t kind;                                    /* MN_HYB_* mixer */
+  int32_t heads, kv_heads, dim, vdim;              /* lightning, gla: kv_heads = heads; talk attention: vdim = dim (the values are the projected keys) */
   int32_t ff_kind;                                 /* MN_HYB_FF_* */
   int32_t ff;                                      /* dense: the feed-forward's width; moe: the shared expert's (0: none) */
+  int32_t ff_act;                                  /* MN_HYB_ACT_* */
   int32_t experts, pass, top, expert_ff;           /* moe: the router has experts + pass outputs, the last `pass` stand for the input itself */
+  int32_t expert_glu;                              /* moe: 0 = W_down relu(W_up h)^2, 1 = W_down (silu(W_gate h) * W_up h) */
   int32_t temp_every;                              /* attention: 0 = no query temperature */
+  int32_t rot_dims, window, chunk;                 /* talk attention (0: none) */
+  int32_t conv;                                    /* channel delta: taps of the q / k / v filters */
+  int32_t rank_a, rank_g;                          /* channel delta, gla: rank of the decay projection; channel delta: of the gate projection */
   float scale, temp_coef;
-  const float* sink;                               /* attention: DEVICE fp32 [heads] or NULL */
+  float act_pos, act_neg;                          /* xielu: the factors of its two branches */
+  float unit_eps;                                  /* channel delta: inside the root of the unit norms */
+  float root;                                      /* gla: exponent of the decays' sigmoid */
+  const float* sink;                               /* attention, talk attention: DEVICE fp32 [heads] or NULL */
   const float* decay;                              /* lightning: DEVICE fp32 [heads] */
   const float* correction;                         /* moe: DEVICE fp32 [experts + pass] or NULL */
+  const float* talk;                               /* talk attention: DEVICE fp32 [heads, heads] */
+  const float* rot_freq;                           /* talk attention: DEVICE fp32 [rot_dims / 2] */
+  const float* a_log;                              /* channel delta: DEVICE fp32 [heads] */
+  const int32_t* table;                            /* moe: DEVICE int32 [vocab, top]: the experts by token id, each with weight 1 / top (no router rows) */
   const uint16_t *norm1;                           /* [width] */
   const uint16_t *q_norm, *k_norm;                 /* attention: [dim] */
-  const uint16_t *mix_norm;                        /* lightning: [heads * vdim] */
-  const uint16_t *w_in;                            /* rows [q ; k ; v ; (lightning: gate) ; up of the dense or shared expert ; router ; zero rows up to a multiple of 8] x width */
+  const uint16_t *mix_norm;                        /* lightning: [heads * vdim]; channel delta, gla: [vdim] */
+  const uint16_t *w_conv;                          /* channel delta: [2 kv_heads dim + heads vdim, conv] */
+  const uint16_t *w_a2, *b_a2;                     /* channel delta, gla: [heads dim, rank_a], bias [heads dim] */
+  const uint16_t *w_g2;                            /* channel delta: [heads vdim, rank_g] */
+  const uint16_t *w_in;                            /* rows [mixer ; up of the dense or shared expert ; router ; zero rows up to a multiple of 8] x width with the mixer's rows
+                                                    * attention [q ; k ; v], lightning [q ; k ; v ; gate], talk attention [q ; k], channel delta [q ; k ; v ; a1 ; g1 ; b], gla [q ; k ; v ; gate ; a1] */
   const uint16_t *w_out;                           /* [width, heads * vdim + ff] = [mixer o | down of the dense or shared expert] */
-  const uint16_t *w_up;                            /* moe: [experts, expert_ff, width] */
+  const uint16_t *w_up;                            /* moe: [experts, expert_ff, width]; expert_glu: [experts, 2 expert_ff, width] = [gate ; up] */
   const uint16_t *w_down;                          /* moe: [experts, width, expert_ff] */
 } mn_hyb_layer;
 typedef struct mn_hyb_model {
   int32_t width, n_layers, n_runs, arith;
+  int32_t norm;                                    /* MN_HYB_NORM_* of norm1 and the final norm */
+  int32_t vocab;                                   /* rows of the layers' tables */
+  int32_t block_rows;                              /* rows per run of the caller's blk_tab (talk attention) */
   float eps;
   const mn_hyb_layer* layers;                      /* HOST array [n_layers] */
   const int32_t* run_layer;                        /* HOST [n_runs]: the layer of every run */
@@ -1135,7 +1162,8 @@ typedef struct mn_hyb_model {
 typedef struct mn_hyb_state {                      /* HOST arrays [n_runs] of device pointers, fp32 */
   float* const* k;                                 /* attention runs: [n_seq, t_max, kv_heads * dim] */
   float* const* v;                                 /* attention runs: [n_seq, t_max, kv_heads * vdim] */
-  float* const* lin;                               /* lightning runs: [n_seq, heads, dim, vdim] */
+  float* const* lin;                               /* runs with a recurrence: [n_seq, heads, dim, vdim] */
+  float* const* conv;                              /* channel delta runs: [n_seq, conv - 1, 2 kv_heads dim + heads vdim] */
   int32_t n_seq, t_max;
 } mn_hyb_state;
 MN_API size_t mn_sizeof_hyb_layer(void);
@@ -1143,11 +1171,12 @@ MN_API size_t mn_sizeof_hyb_model(void);
 MN_API size_t mn_sizeof_hyb_state(void);
 /* One pass of the stack over M rows; rows, row arrays, blk_tab / n_blk, max_len, flags, out and trace as mn_pmix_step (trace: fp32
  * [n_runs, M, width]).  chunk_tab / n_chunks: the rows cut into chunks of <= mn_lightning_chunk_rows() consecutive rows of one
- * sequence (NULL / 0: the recurrences walk their rows one by one). */
+ * sequence (NULL / 0: the recurrences walk their rows one by one).  row_tok int32 [M]: the rows' token ids (read by layers with a table). */
 MN_API size_t mn_hyb_workspace_bytes(const mn_hyb_model* m, int M);
-MN_API int mn_hyb_step(const mn_hyb_model* m, const mn_hyb_state* st, const float* x, int64_t ldx, int M, const int32_t* row_seq,
-                       const int32_t* row_slot, const int32_t* row_back, const int32_t* blk_tab, int n_blk, const int32_t* chunk_tab,
-                       int n_chunks, int max_len, int flags, float* out, float* trace, void* workspace, size_t workspace_bytes, void* stream);
+MN_API int mn_hyb_step(const mn_hyb_model* m, const mn_hyb_state* st, const float* x, int64_t ldx, int M, const int32_t* row_tok,
+                       const int32_t* row_seq, const int32_t* row_slot, const int32_t* row_back, const int32_t* blk_tab, int n_blk,
+                       const int32_t* chunk_tab, int n_chunks, int max_len, int flags, float* out, float* trace, void* workspace,
+                       size_t workspace_bytes, void* stream);
 
 /* The block attention of section 10 with a sink per head (or NULL), a soft cap of the scores (softcap > 0: every score s becomes
  * softcap * tanh(s / softcap) before the softmax; 0: none) and explicit row strides of the two arenas (ldk, ldv in floats; 0 = G * dim,
@@ -1278,6 +1307,69 @@ MN_API size_t mn_pn_workspace_bytes(const mn_pn_model* m, int M);
 MN_API int mn_pn_step(const mn_pn_model* m, const mn_pn_state* st, const float* x, int64_t ldx, int M, const int32_t* row_tok,
                       const int32_t* row_seq, const int32_t* row_slot, const int32_t* row_back, const int32_t* blk_tab, int n_blk, int max_len,
                       int flags, float* out, float* trace, void* workspace, size_t workspace_bytes, void* stream);
+
+/* ------------------------------------------------------------------------------------------
+ * 13. Layers with a decay per key channel and mixed attention heads (0.1.30): further mixers of the hybrid step function (section 11) —
+ *     the delta rule with one decay per head and KEY CHANNEL (MN_HYB_CHANNEL_DELTA), gated linear attention (MN_HYB_GLA: the same state
+ *     with a plain k v^T write), and softmax attention whose heads' scores are mixed by a matrix before the softmax, over chunks of
+ *     positions, with values that are the projected keys (MN_HYB_TALK_ATTENTION) — with LayerNorm instead of RMS norm, the xIELU
+ *     activation, silu-gated experts, and experts chosen by a table over token ids.  Norms, angles, scores, softmax, decays, gates and the
+ *     recurrent state are fp32 in both arithmetic modes.
+ * ------------------------------------------------------------------------------------------ */
+/* x += y (optional) + sum_j w_j ye[r(m, j)] (top > 0; r as in mn_moe_combine_residual, w_j = ew[m top + j], or ew_all for all when ew is
+ * NULL); then, with w: n = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w into h (fp32) and / or h16 (bf16). */
+MN_API int mn_add_layernorm_rows(float* x, int64_t ldx, const float* y, int64_t ldy, const float* ye, int64_t ldye, const int32_t* slot_of,
+                                 const float* ew, float ew_all, int top, const uint16_t* w, float eps, float* h, int64_t ldh, uint16_t* h16,
+                                 int64_t ldh16, int M, int n, void* stream);
+/* y = alpha_pos z^2 + z / 2 where z > 0, alpha_neg (exp(z) - 1 - z) + z / 2 elsewhere; y16: optional bf16 copy */
+MN_API int mn_xielu_rows(const float* x, int64_t ldx, float alpha_pos, float alpha_neg, float* y, int64_t ldy, uint16_t* y16, int64_t ldy16,
+                         int M, int n, void* stream);
+/* idx[m, j] = table[tok[m], j], table int32 [vocab, top] (a token id outside it reads the nearest row); w (fp32 [M, top] or NULL) = 1 / top */
+MN_API int mn_token_table_rows(const int32_t* table, int vocab, int top, const int32_t* tok, int M, int32_t* idx, float* w, void* stream);
+/* Second stage of a low-rank projection with the function behind it: z = w a + bias (w bf16 [n, k], a the k values at a + m * lda, bias bf16
+ * [n] or NULL), out[m, c] = z (LINEAR), exp(-exp(a_log[c / head_n]) softplus(z)) (DECAY), sigmoid(z)^root (ROOT) or sigmoid(z) (SIGMOID).
+ * One or two jobs share the launch. */
+enum { MN_LOW_RANK_LINEAR = 0, MN_LOW_RANK_DECAY = 1, MN_LOW_RANK_ROOT = 2, MN_LOW_RANK_SIGMOID = 3 };
+typedef struct mn_low_rank_job {
+  const float* a; int64_t lda;
+  const uint16_t *w, *bias;
+  const float* a_log;                              /* DECAY: DEVICE fp32 [n / head_n] */
+  float* out; int64_t ldo;
+  int32_t k, n, kind, head_n;
+  float root;
+} mn_low_rank_job;
+MN_API int mn_low_rank_gate_rows(const mn_low_rank_job* jobs, int n_jobs, int M, void* stream);
+/* Recurrence with a decay per key channel over each sequence's rows, per head h (q / k head h / (H / G)): S <- diag(g) S with g = the row's
+ * dim decays of the head (g fp32 [M, H dim]); then with beta (fp32 [M, H]) the delta rule's write u = beta (v - S^T k), S <- S + k u^T,
+ * with beta NULL the plain write S <- S + k v^T; out[m, h vdim + c] = o_scale (S^T q)[c].  qkv fp32 [M, ld] = [q: G dim ; k: G dim ; v: H
+ * vdim]; state fp32 [n_seq, H, dim, vdim] (a row at slot 0 starts from zero) is left at the sequence's last row.  Rows of one sequence
+ * are consecutive (row_back as in section 9); blk_tab (optional): the runs of rows, whose firsts include every sequence's first row.
+ * flags: MN_SEQ_ROWS_DISTINCT = every row is alone in its sequence (a decode step).  dim <= 4096. */
+MN_API int mn_channel_state_rows(const float* qkv, int64_t ld, const float* g, int64_t ldg, const float* beta, int64_t ldb, int M, int H, int G,
+                                 int dim, int vdim, float o_scale, float* state, const int32_t* row_seq, const int32_t* row_slot,
+                                 const int32_t* row_back, const int32_t* blk_tab, int n_blk, int flags, float* out, int64_t ldo, void* stream);
+/* mn_head_rms_silu_gate_rows with the gate's function named: the gate as it is, through silu, or through a sigmoid */
+enum { MN_GATE_ACT_NONE = 0, MN_GATE_ACT_SILU = 1, MN_GATE_ACT_SIGMOID = 2 };
+MN_API int mn_head_rms_gate_rows(const float* x, int64_t ldx, const uint16_t* w, float eps, const float* g, int64_t ldg, int act, float* y,
+                                 int64_t ldy, uint16_t* y16, int64_t ldy16, int M, int H, int vdim, void* stream);
+/* C[z, n] = silu(W_i[n] . a) * (W_i[N + n] . a) with i = w_idx[z] (rows of an i outside [0, n_idx) are left as they are), a = A + (z / a_div) * lda */
+MN_API int mn_gemv_glu_indexed(const float* A, int64_t lda, int a_div, const uint16_t* W, int64_t ldw, int64_t w_bs, const int32_t* w_idx,
+                               int n_idx, float* C, int64_t ldc, int Z, int N, int K, void* stream);
+/* Softmax attention with mixed heads: score_h = sum_g talk[h, g] (q_g . k_(g / (H / G))) (q fp32 [M, H dim], scaled by the caller; talk DEVICE
+ * fp32 [H, H]) over the keys j of the row's sequence with j <= pos, pos - j < window (window > 0) and floor(j / chunk) = floor(pos / chunk)
+ * (chunk > 0), softmax with exp(sink[h]) added to the denominator (sink DEVICE fp32 [H] or NULL), values of key/value head h / (H / G)
+ * with dim values; arenas [n_seq, t_max, ld].  blk_tab int32 [n_blk, 2]: runs of <= rows consecutive rows of one sequence (NULL: every
+ * row is a run, rows = 1, n_blk = M).  rows: at most mn_talk_attn_block_rows(H, G, dim) for the matrix-core kernel (0: no instance; the
+ * plain kernel takes H <= 112, H dim <= 16384).  nsplit key splits (mn_talk_attn_splits proposes) with a workspace and a merge launch.
+ * variant -1: the matrix-core kernel where it has an instance. */
+enum { MN_TALK_ATTN_MFMA = 0, MN_TALK_ATTN_PLAIN = 1 };
+MN_API int mn_talk_attn_block_rows(int H, int G, int dim);
+MN_API int mn_talk_attn_splits(int n_blk, int max_keys);
+MN_API size_t mn_talk_attn_workspace_bytes(int n_blk, int H, int G, int dim, int rows, int nsplit);
+MN_API int mn_talk_attn(const float* q, int64_t ldq, const float* k_arena, int64_t ldk, const float* v_arena, int64_t ldv, const float* talk,
+                        const float* sink, const int32_t* row_seq, const int32_t* row_slot, int M, const int32_t* blk_tab, int n_blk, int rows,
+                        int H, int G, int dim, int t_max, int window, int chunk, float* out, int64_t ldo, uint16_t* out16, int64_t ldo16,
+                        int nsplit, void* workspace, size_t workspace_bytes, int variant, void* stream);
 
 #ifdef __cplusplus
 }

@@ -144,19 +144,25 @@ class PmixState(C.Structure):
 
 
 class HybLayer(C.Structure):
-    _fields_ = [(k, C.c_int32) for k in ("kind", "heads", "kv_heads", "dim", "vdim", "ff_kind", "ff", "experts", "n_pass", "top", "expert_ff",
-                                         "temp_every")] + \
-               [(k, C.c_float) for k in ("scale", "temp_coef")] + \
-               [(k, C.c_void_p) for k in ("sink", "decay", "correction", "norm1", "q_norm", "k_norm", "mix_norm", "w_in", "w_out", "w_up", "w_down")]
+    _fields_ = [(k, C.c_int32) for k in ("kind", "heads", "kv_heads", "dim", "vdim", "ff_kind", "ff", "ff_act", "experts", "n_pass", "top",
+                                         "expert_ff", "expert_glu", "temp_every", "rot_dims", "window", "chunk", "conv", "rank_a", "rank_g")] + \
+               [(k, C.c_float) for k in ("scale", "temp_coef", "act_pos", "act_neg", "unit_eps", "root")] + \
+               [(k, C.c_void_p) for k in ("sink", "decay", "correction", "talk", "rot_freq", "a_log", "table", "norm1", "q_norm", "k_norm",
+                                          "mix_norm", "w_conv", "w_a2", "b_a2", "w_g2", "w_in", "w_out", "w_up", "w_down")]
 
 
 class HybModel(C.Structure):
-    _fields_ = [("width", C.c_int32), ("n_layers", C.c_int32), ("n_runs", C.c_int32), ("arith", C.c_int32), ("eps", C.c_float),
-                ("layers", C.POINTER(HybLayer)), ("run_layer", C.POINTER(C.c_int32)), ("final_w", C.c_void_p)]
+    _fields_ = [(k, C.c_int32) for k in ("width", "n_layers", "n_runs", "arith", "norm", "vocab", "block_rows")] + \
+               [("eps", C.c_float), ("layers", C.POINTER(HybLayer)), ("run_layer", C.POINTER(C.c_int32)), ("final_w", C.c_void_p)]
 
 
 class HybState(C.Structure):
-    _fields_ = [(k, PP) for k in ("k", "v", "lin")] + [("n_seq", C.c_int32), ("t_max", C.c_int32)]
+    _fields_ = [(k, PP) for k in ("k", "v", "lin", "conv")] + [("n_seq", C.c_int32), ("t_max", C.c_int32)]
+
+
+class LowRankJob(C.Structure):
+    _fields_ = [("a", C.c_void_p), ("lda", C.c_int64), ("w", C.c_void_p), ("bias", C.c_void_p), ("a_log", C.c_void_p), ("out", C.c_void_p),
+                ("ldo", C.c_int64), ("k", C.c_int32), ("n", C.c_int32), ("kind", C.c_int32), ("head_n", C.c_int32), ("root", C.c_float)]
 
 
 class PnLayer(C.Structure):
@@ -389,7 +395,7 @@ SYMBOLS = {
     "mn_router_softmax_topk_rows": (_i, [_p, _i64, _i, _i, _i, _i, _p, _p, _p, _p, _i64, _p, _i64, _i, _p]),
     "mn_moe_combine_pass_residual": (_i, [_p, _i64, _p, _i64, _p, _p, _p, _i, _i, _p, _i64, _p, _i64, _i, _i, _p]),
     "mn_hyb_workspace_bytes": (_sz, [C.POINTER(HybModel), _i]),
-    "mn_hyb_step": (_i, [C.POINTER(HybModel), C.POINTER(HybState), _p, _i64, _i, _p, _p, _p, _p, _i, _p, _i, _i, _i, _p, _p, _p, _sz, _p]),
+    "mn_hyb_step": (_i, [C.POINTER(HybModel), C.POINTER(HybState), _p, _i64, _i, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _p, _p, _p, _sz, _p]),
     # section 12: post-norm mixed-mixer sequence models
     "mn_window_pool_attn_blocks_cap": (_i, [_p, _i64, _p, _i64, _p, _i64, _p, _p, _p, _f, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f,
                                             _p, _i64, _p, _i64, _i, _p, _sz, _i, _p]),
@@ -406,6 +412,20 @@ SYMBOLS = {
     "mn_head_rms_silu_gate_rows": (_i, [_p, _i64, _p, _f, _p, _i64, _p, _i64, _p, _i64, _i, _i, _i, _p]),
     "mn_pn_workspace_bytes": (_sz, [C.POINTER(PnModel), _i]),
     "mn_pn_step": (_i, [C.POINTER(PnModel), C.POINTER(PnState), _p, _i64, _i, _p, _p, _p, _p, _p, _i, _i, _i, _p, _p, _p, _sz, _p]),
+    # section 13: decays per key channel, mixed attention heads
+    "mn_rope_unit_append_from": (_i, [_p, _i64, _i, _i, _i, _i, _i, _i, _i, _p, _f, _i, _f, _f, _p, _p, _p, _i64, _p, _p, _i, _p]),
+    "mn_add_layernorm_rows": (_i, [_p, _i64, _p, _i64, _p, _i64, _p, _p, _f, _i, _p, _f, _p, _i64, _p, _i64, _i, _i, _p]),
+    "mn_xielu_rows": (_i, [_p, _i64, _f, _f, _p, _i64, _p, _i64, _i, _i, _p]),
+    "mn_token_table_rows": (_i, [_p, _i, _i, _p, _i, _p, _p, _p]),
+    "mn_low_rank_gate_rows": (_i, [C.POINTER(LowRankJob), _i, _i, _p]),
+    "mn_channel_state_rows": (_i, [_p, _i64, _p, _i64, _p, _i64, _i, _i, _i, _i, _i, _f, _p, _p, _p, _p, _p, _i, _i, _p, _i64, _p]),
+    "mn_head_rms_gate_rows": (_i, [_p, _i64, _p, _f, _p, _i64, _i, _p, _i64, _p, _i64, _i, _i, _i, _p]),
+    "mn_gemv_glu_indexed": (_i, [_p, _i64, _i, _p, _i64, _i64, _p, _i, _p, _i64, _i, _i, _i, _p]),
+    "mn_talk_attn_block_rows": (_i, [_i, _i, _i]),
+    "mn_talk_attn_splits": (_i, [_i, _i]),
+    "mn_talk_attn_workspace_bytes": (_sz, [_i, _i, _i, _i, _i, _i]),
+    "mn_talk_attn": (_i, [_p, _i64, _p, _i64, _p, _i64, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p, _i64, _p, _i64, _i, _p, _sz,
+                          _i, _p]),
     "mn_semdec_step": (_i, [C.POINTER(SemDec), _p, _i, _p, _p, _p, _p, _i, _i64, _p, _p, _p, _sz, _p]),
 }
 
@@ -426,7 +446,7 @@ def lib():
         fn = getattr(handle, name)  # AttributeError if the symbol is missing
         fn.restype = res
         fn.argtypes = args
-    if handle.mn_version() < 129:
+    if handle.mn_version() < 130:
         raise RuntimeError("libmingnative.so is too old")
     check_struct_layouts(handle)
     _lib = handle

@@ -701,6 +701,112 @@ def daberax_param_shapes(cfg: DaberaxConfig):
     return s
 
 
+# ---- Sabezen ---------------------------------------------------------------------------------------------------------------
+SABEZEN_MIXERS = ("attention", "channel_delta", "gla")
+
+
+class SabezenConfig(_Config):
+    """A stack of layers that run their mixer and their feed-forward in parallel on one layer-normed input.  `layers` is a list of
+    dicts(type, mixer, mlp):
+    type  "attention":     mixer dict(heads, kv_heads, dim, vdim = dim, scale, optional rot dict(base, dims), optional mask dict(size)): the
+                           values are the projected keys, rotary half pairs then a unit RMS per head, the heads' scores mixed by a
+                           matrix, chunks of mask.size positions that see only themselves, one added to the softmax's denominator
+          "channel_delta": mixer dict(heads, kv_heads, dim, vdim, conv): the delta rule with one decay per head and key channel
+          "gla":           mixer dict(heads, dim, vdim, tau): gated linear attention, decays sigmoid(z)^(1 / tau)
+    mlp   None, dict(kind="dense", ff) (xIELU), or dict(kind="moe", router dict(experts, top), expert dict(ff)): silu-gated experts that a
+          table picks by token id
+    embedding dict(scale): factor of the input embeddings.  The ranks of the low-rank projections come from the tensors' shapes;
+    nothing is assumed equal between layers."""
+    model_type = "sabezen"
+
+    def __init__(self, width=256, vocab=1024, layers=(), norm=None, embedding=None, architecture="Sabezen", **kwargs):
+        self.architecture = architecture
+        self.width, self.vocab = int(width), int(vocab)
+        self.layers = [copy.deepcopy(dict(ly)) for ly in layers]
+        self.norm = dict(norm or {"eps": 1e-6})
+        self.embedding = dict(embedding or {})
+        super().__init__(**kwargs)
+        self.validate()
+
+    eps = property(lambda self: float(self.norm["eps"]))
+    embed_scale = property(lambda self: float(self.embedding.get("scale", 1.0)))
+
+    def validate(self):
+        for i, ly in enumerate(self.layers):
+            t = ly.get("type")
+            if t not in SABEZEN_MIXERS:
+                raise ValueError(f"layer {i}: unknown mixer type {t!r} (known: {SABEZEN_MIXERS})")
+            m = ly["mixer"]
+            need = {"attention": ("heads", "kv_heads", "dim", "scale"), "channel_delta": ("heads", "kv_heads", "dim", "vdim", "conv"),
+                    "gla": ("heads", "dim", "vdim", "tau")}[t]
+            for k in need:
+                if k not in m:
+                    raise ValueError(f"layer {i}: mixer lacks {k!r}")
+            if t != "gla" and int(m["heads"]) % int(m["kv_heads"]):
+                raise ValueError(f"layer {i}: {m['heads']} heads do not divide over {m['kv_heads']} key heads")
+            if t == "channel_delta" and int(m["conv"]) < 1:
+                raise ValueError(f"layer {i}: conv must be >= 1")
+            if t == "gla" and float(m["tau"]) <= 0:
+                raise ValueError(f"layer {i}: tau must be positive")
+            if t == "attention":
+                if int(m.get("vdim", m["dim"])) != int(m["dim"]):
+                    raise ValueError(f"layer {i}: the values are the keys, so vdim = {m['vdim']} must be dim = {m['dim']}")
+                rot = m.get("rot")
+                if rot and (int(rot["dims"]) % 2 or not (0 <= int(rot["dims"]) <= int(m["dim"]))):
+                    raise ValueError(f"layer {i}: rot.dims = {rot['dims']} must be even and at most {m['dim']}")
+                if m.get("mask") and int(m["mask"]["size"]) < 1:
+                    raise ValueError(f"layer {i}: mask.size must be >= 1")
+            mlp = ly.get("mlp")
+            if mlp is None:
+                continue
+            if mlp.get("kind") == "dense":
+                if int(mlp["ff"]) < 1:
+                    raise ValueError(f"layer {i}: dense feed-forward needs ff >= 1")
+            elif mlp.get("kind") == "moe":
+                r = mlp["router"]
+                if not (1 <= int(r["top"]) <= int(r["experts"])):
+                    raise ValueError(f"layer {i}: router {r}: 1 <= top <= experts")
+            else:
+                raise ValueError(f"layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
+
+
+def sabezen_param_shapes(cfg: SabezenConfig, ranks):
+    """{tensor name: shape} of a Sabezen checkpoint (`l<i>.` per layer, `mix.` the mixer's and `mlp.` the feed-forward's tensors; the `table`s
+    are integers).  ranks(name) -> rows of the first stage of a low-rank projection (`l<i>.mix.a1`, `l<i>.mix.g1`)."""
+    W, V = cfg.width, cfg.vocab
+    s = {"embed": (V, W)}
+    for i, ly in enumerate(cfg.layers):
+        p, m, mlp, t = f"l{i}.", ly["mixer"], ly.get("mlp"), ly["type"]
+        H, d = int(m["heads"]), int(m["dim"])
+        e = int(m.get("vdim", d))
+        s[p + "norm1"] = (W,)
+        if t == "attention":
+            s[p + "mix.q"], s[p + "mix.k"], s[p + "mix.talk"] = (H * d, W), (int(m["kv_heads"]) * d, W), (H, H)
+        elif t == "channel_delta":
+            G, taps, ra, rg = int(m["kv_heads"]), int(m["conv"]), ranks(p + "mix.a1"), ranks(p + "mix.g1")
+            for n, rows in (("q", G * d), ("k", G * d), ("v", H * e)):
+                s[p + "mix." + n], s[p + "mix." + n + ".conv"] = (rows, W), (rows, taps)
+            s[p + "mix.b"], s[p + "mix.A_log"], s[p + "mix.dt_bias"], s[p + "mix.norm"] = (H, W), (H,), (H * d,), (e,)
+            s[p + "mix.a1"], s[p + "mix.a2"], s[p + "mix.g1"], s[p + "mix.g2"] = (ra, W), (H * d, ra), (rg, W), (H * e, rg)
+        else:
+            ra = ranks(p + "mix.a1")
+            s[p + "mix.q"], s[p + "mix.k"], s[p + "mix.v"], s[p + "mix.g"] = (H * d, W), (H * d, W), (H * e, W), (H * e, W)
+            s[p + "mix.a1"], s[p + "mix.a2"], s[p + "mix.a2.b"], s[p + "mix.norm"] = (ra, W), (H * d, ra), (H * d,), (e,)
+        s[p + "mix.o"] = (W, H * e)
+        if mlp is None:
+            continue
+        if mlp["kind"] == "dense":
+            ff = int(mlp["ff"])
+            s[p + "mlp.up"], s[p + "mlp.down"], s[p + "mlp.act"] = (ff, W), (W, ff), (2,)
+        else:
+            ff = int(mlp["expert"]["ff"])
+            for j in range(int(mlp["router"]["experts"])):
+                s[f"{p}mlp.e{j}.gate"], s[f"{p}mlp.e{j}.up"], s[f"{p}mlp.e{j}.down"] = (ff, W), (ff, W), (W, ff)
+            s[p + "mlp.table"] = (V, int(mlp["router"]["top"]))
+    s["final.norm"], s["head"] = (W,), (V, W)
+    return s
+
+
 # ---- registry: which configuration class a config.json belongs to -------------------------------------------------------------
 def _is_pizitar(d):
     return d.get("architecture") == "Pizitar" or d.get("model_type") == "pizitar"
@@ -718,12 +824,16 @@ def _is_daberax(d):
     return d.get("architecture") == "Daberax" or d.get("model_type") == "daberax"
 
 
+def _is_sabezen(d):
+    return d.get("architecture") == "Sabezen" or d.get("model_type") == "sabezen"
+
+
 def _is_ming_univision(d):
     return "llm_config" in d or d.get("model_type") in ("bailingmm", "ming_univision")
 
 
 MODEL_REGISTRY = [("pizitar", _is_pizitar, PizitarConfig), ("sakinex", _is_sakinex, SakinexConfig), ("zuzenex", _is_zuzenex, ZuzenexConfig),
-                  ("daberax", _is_daberax, DaberaxConfig),
+                  ("daberax", _is_daberax, DaberaxConfig), ("sabezen", _is_sabezen, SabezenConfig),
                   ("ming_univision", _is_ming_univision, MingUniVisionConfig)]
 
 

@@ -148,18 +148,20 @@ extern "C" int mn_struct_layout(int which, size_t* offsets, int cap) {
   };
   static const size_t hyb_layer[] = {
 #define F(f) MN_OFF(mn_hyb_layer, f)
-      F(kind) F(heads) F(kv_heads) F(dim) F(vdim) F(ff_kind) F(ff) F(experts) F(pass) F(top) F(expert_ff) F(temp_every) F(scale) F(temp_coef)
-      F(sink) F(decay) F(correction) F(norm1) F(q_norm) F(k_norm) F(mix_norm) F(w_in) F(w_out) F(w_up) F(w_down)
+      F(kind) F(heads) F(kv_heads) F(dim) F(vdim) F(ff_kind) F(ff) F(ff_act) F(experts) F(pass) F(top) F(expert_ff) F(expert_glu)
+      F(temp_every) F(rot_dims) F(window) F(chunk) F(conv) F(rank_a) F(rank_g) F(scale) F(temp_coef) F(act_pos) F(act_neg) F(unit_eps)
+      F(root) F(sink) F(decay) F(correction) F(talk) F(rot_freq) F(a_log) F(table) F(norm1) F(q_norm) F(k_norm) F(mix_norm) F(w_conv)
+      F(w_a2) F(b_a2) F(w_g2) F(w_in) F(w_out) F(w_up) F(w_down)
 #undef F
   };
   static const size_t hyb_model[] = {
 #define F(f) MN_OFF(mn_hyb_model, f)
-      F(width) F(n_layers) F(n_runs) F(arith) F(eps) F(layers) F(run_layer) F(final_w)
+      F(width) F(n_layers) F(n_runs) F(arith) F(norm) F(vocab) F(block_rows) F(eps) F(layers) F(run_layer) F(final_w)
 #undef F
   };
   static const size_t hyb_state[] = {
 #define F(f) MN_OFF(mn_hyb_state, f)
-      F(k) F(v) F(lin) F(n_seq) F(t_max)
+      F(k) F(v) F(lin) F(conv) F(n_seq) F(t_max)
 #undef F
   };
   static const size_t pn_layer[] = {

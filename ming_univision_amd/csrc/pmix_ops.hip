@@ -244,6 +244,7 @@ struct RopeArgs {
   const int32_t* row_seq; const int32_t* row_slot;
   float* q_out; int64_t ldq;
   float* k_arena; float* v_arena; int t_max;
+  int v_col;                                    // column of the first value head in a row
   // decode rows only (ROW): the channel filter in front with its state, and the block means behind
   const bf16_t* w_conv; int conv; float* conv_state;
   float* pk; float* pv; int n_pool_max, pool;
@@ -305,7 +306,7 @@ __global__ __launch_bounds__(256) void rope_unit_append_kernel(RopeArgs a, int M
   };
   if (hv >= a.H + a.G) {                                         // a value head: into its arena
     const int g = hv - a.H - a.G;
-    for (int i = lane; i < a.vdim; i += 64) put(a.v_arena, a.pv, a.G * a.vdim, g * a.vdim + i, ld((a.H + a.G) * a.dim + g * a.vdim + i));
+    for (int i = lane; i < a.vdim; i += 64) put(a.v_arena, a.pv, a.G * a.vdim, g * a.vdim + i, ld(a.v_col + g * a.vdim + i));
     return;
   }
   const bool is_q = hv < a.H;
@@ -1121,11 +1122,18 @@ extern "C" int mn_axpy_rms_filter_rows(float* x, int64_t ldx, const float* y, in
 extern "C" int mn_rope_unit_append(const float* qkv, int64_t ldqkv, int M, int H, int G, int dim, int vdim, int rot_dims, const float* freq,
                                    float mag, int unit, float eps, float q_scale, const int32_t* row_seq, const int32_t* row_slot,
                                    float* q_out, int64_t ldq, float* k_arena, float* v_arena, int t_max, void* stream) {
-  MN_CHECK_ARG(qkv && row_seq && row_slot && q_out && k_arena && v_arena && M >= 1 && M <= 65535 && H >= 1 && G >= 1 && t_max >= 1,
+  return mn_rope_unit_append_from(qkv, ldqkv, M, H, G, dim, vdim, (H + G) * dim, rot_dims, freq, mag, unit, eps, q_scale, row_seq, row_slot, q_out,
+                                  ldq, k_arena, v_arena, t_max, stream);
+}
+
+extern "C" int mn_rope_unit_append_from(const float* qkv, int64_t ldqkv, int M, int H, int G, int dim, int vdim, int v_col, int rot_dims,
+                                        const float* freq, float mag, int unit, float eps, float q_scale, const int32_t* row_seq,
+                                        const int32_t* row_slot, float* q_out, int64_t ldq, float* k_arena, float* v_arena, int t_max, void* stream) {
+  MN_CHECK_ARG(qkv && row_seq && row_slot && q_out && k_arena && v_arena && M >= 1 && M <= 65535 && H >= 1 && G >= 1 && t_max >= 1 && v_col >= 0,
                "mn_rope_unit_append: bad args");
   MN_CHECK_ARG(dim >= 1 && dim <= 512 && vdim >= 1 && rot_dims >= 0 && rot_dims <= dim && (rot_dims % 2) == 0 && (rot_dims == 0 || freq),
                "mn_rope_unit_append: dim=%d (at most 512), rot_dims=%d (even, at most dim)", dim, rot_dims);
-  RopeArgs a{qkv, ldqkv, H, G, dim, vdim, rot_dims, freq, mag, unit, eps, q_scale, row_seq, row_slot, q_out, ldq, k_arena, v_arena, t_max,
+  RopeArgs a{qkv, ldqkv, H, G, dim, vdim, rot_dims, freq, mag, unit, eps, q_scale, row_seq, row_slot, q_out, ldq, k_arena, v_arena, t_max, v_col,
              nullptr, 0, nullptr, nullptr, nullptr, 0, 0, nullptr, 0, nullptr, 0, nullptr, 0, 0.f, nullptr, 0};
   hipLaunchKernelGGL((rope_unit_append_kernel<false>), dim3((unsigned)mn_cdiv(H + 2 * G, 4), (unsigned)M), dim3(256), 0, mn_stream(stream), a, M);
   MN_CHECK_LAUNCH("mn_rope_unit_append");
@@ -1146,7 +1154,7 @@ extern "C" int mn_filter_rope_append_rows(const float* qkv, int64_t ldqkv, int M
   MN_CHECK_ARG(conv >= 0 && (conv == 0 || w_conv) && (conv <= 1 || conv_state) && pool >= 0 && (pool == 0 || (pk && pv && n_pool_max >= 1)),
                "mn_filter_rope_append_rows: bad filter or block arenas");
   RopeArgs a{qkv, ldqkv, H, G, dim, vdim, rot_dims, freq, mag, unit, eps, q_scale, row_seq, row_slot, q_out, ldq, k_arena, v_arena, t_max,
-             w_conv, conv, conv_state, pk, pv, n_pool_max, pool, zx, ldzx, g, ldg, gru_state, gru_n, gru_scale, gru_out, ldgo};
+             (H + G) * dim, w_conv, conv, conv_state, pk, pv, n_pool_max, pool, zx, ldzx, g, ldg, gru_state, gru_n, gru_scale, gru_out, ldgo};
   hipLaunchKernelGGL((rope_unit_append_kernel<true>), dim3((unsigned)(mn_cdiv(H + 2 * G, 4) + mn_cdiv(gru_n, 256)), (unsigned)M), dim3(256), 0,
                      mn_stream(stream), a, M);
   MN_CHECK_LAUNCH("mn_filter_rope_append_rows");

@@ -11,6 +11,7 @@
 #include <math.h>
 
 #include "common.h"
+#include "delta_device.h"
 #include "mfma_f32_tiles.h"
 
 extern "C" int mn_rotary_frequencies_scaled_host(int dims, double base, double factor, double low, double high, double original, float* freq) {
@@ -33,10 +34,6 @@ extern "C" int mn_rotary_frequencies_scaled_host(int dims, double base, double f
 }
 
 namespace {
-
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float silu_x(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 
 // ---------------------------------------------------------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void rms_scale_add_kernel(float* __restrict__ x, int64_t ldx, const float* __restrict__ y, int64_t ldy,
@@ -204,66 +201,10 @@ __global__ __launch_bounds__(256) void head_sigmoid_gate_kernel(float* __restric
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------
-// Gated delta rule, preparation of a row: channels [q: G dim ; k: G dim ; v: H vdim] of the raw projections go through their causal
-// filter (earlier inputs from the rows before it in this call, then from the sequence's state) and silu; q and k heads become unit
-// vectors (q also times q_scale); beta = sigmoid(b), decay = exp(-exp(a_log) softplus(a + dt_bias)).
-struct DeltaPrepArgs {
-  const float* proj; int64_t ld;             // raw [q ; k ; v] at column 0, b at off_b, a at off_a
-  int H, G, dim, vdim, taps, off_b, off_a;
-  const bf16_t* w_conv;                      // [2 G dim + H vdim, taps], the last tap multiplies the current row
-  float* state;                              // [n_seq, taps - 1, channels]
-  int advance;                               // 1: every row is alone in its sequence and moves the state on by itself
-  const float *a_log, *dt_bias;              // device fp32 [H]
-  float unit_eps, q_scale;
-  const int32_t *row_seq, *row_slot, *row_back;
-  float* qkv; int64_t ldo;                   // [M, channels]
-  float* bd; int64_t ldbd;                   // [M, 2 H]: beta, decay
-};
-
-__device__ __forceinline__ float conv_silu(const DeltaPrepArgs& a, int m, int c, int n, int seq, int slot, int back) {
-  float acc = 0.f;
-  for (int k = 0; k < a.taps; ++k) {
-    float v = 0.f;
-    if (k <= back) v = a.proj[(int64_t)(m - k) * a.ld + c];
-    else if (slot - k >= 0) v = a.state[((int64_t)seq * (a.taps - 1) + (k - back - 1)) * n + c];
-    acc = fmaf(bf16_to_f32(a.w_conv[(int64_t)c * a.taps + (a.taps - 1 - k)]), v, acc);
-  }
-  if (a.advance && a.taps > 1) {                // a one-row sequence: entry i becomes entry i - 1, entry 0 this row's input
-    float* st = a.state + (int64_t)seq * (a.taps - 1) * n + c;
-    for (int i = a.taps - 2; i >= 1; --i) st[(int64_t)i * n] = st[(int64_t)(i - 1) * n];
-    st[0] = a.proj[(int64_t)m * a.ld + c];
-  }
-  return silu_x(acc);
-}
-
 // grid (M, ceil(units / 4)): a wave takes one unit of a row — a q or k head (its unit norm is a wave's reduction) or 256 value channels
 __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrepArgs a) {
-  const int m = blockIdx.x, tid = threadIdx.x, lane = tid & 63, unit = blockIdx.y * 4 + (tid >> 6);
-  const int nqk = 2 * a.G * a.dim, nv = a.H * a.vdim, n = nqk + nv;
-  const int seq = a.row_seq[m], slot = a.row_slot[m], back = a.row_back[m];
-  float* out = a.qkv + (int64_t)m * a.ldo;
-  if (unit < 2 * a.G) {
-    const int c0 = unit * a.dim;
-    float ss = 0.f;
-    for (int d = lane; d < a.dim; d += 64) {
-      const float v = conv_silu(a, m, c0 + d, n, seq, slot, back);
-      out[c0 + d] = v;
-      ss = fmaf(v, v, ss);
-    }
-    ss = wave_sum(ss);
-    const float r = (unit < a.G ? a.q_scale : 1.0f) / sqrtf(ss + a.unit_eps);
-    for (int d = lane; d < a.dim; d += 64) out[c0 + d] *= r;      // the lane rereads what it wrote itself
-  } else {
-    const int e0 = (unit - 2 * a.G) * 256;
-    for (int e = e0 + lane; e < min(nv, e0 + 256); e += 64) out[nqk + e] = conv_silu(a, m, nqk + e, n, seq, slot, back);
-  }
-  if (blockIdx.y == 0) {
-    for (int h = tid; h < a.H; h += 256) {
-      const float* row = a.proj + (int64_t)m * a.ld;
-      a.bd[(int64_t)m * a.ldbd + h] = sigmoid_f(row[a.off_b + h]);
-      a.bd[(int64_t)m * a.ldbd + a.H + h] = expf(-expf(a.a_log[h]) * softplus_f(row[a.off_a + h] + a.dt_bias[h]));
-    }
-  }
+  delta_prep_unit(a, blockIdx.x, blockIdx.y * 4 + (threadIdx.x >> 6), threadIdx.x & 63);
+  if (blockIdx.y == 0) delta_prep_strengths(a, blockIdx.x, threadIdx.x);
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------
@@ -279,13 +220,6 @@ struct DeltaArgs {
   float* out; int64_t ldo;                   // [M, H vdim]
   int M;
 };
-
-__device__ __forceinline__ float sum8(float v) {                    // over the 8 lanes of an aligned group; every lane gets the sum
-  v += dpp_f<0xB1>(v);
-  v += dpp_f<0x4E>(v);
-  v += dpp_f<0x141>(v);
-  return v;
-}
 
 // Rows of sequences (a prompt portion): grid (M, H, ceil(vdim / 32)); the workgroup of a sequence's FIRST row in the call walks that
 // sequence's rows.  A workgroup owns 32 value columns; 8 lanes share a column, lane s of them holds the state rows s, s + 8, ... in
@@ -571,8 +505,9 @@ __global__ __launch_bounds__(256) void delta_step_kernel(DeltaArgs a) {
   }
 }
 
-// grid (ceil(H / 4), M): one wave per head
-__global__ __launch_bounds__(256) void head_rms_silu_gate_kernel(const float* __restrict__ x, int64_t ldx, const bf16_t* __restrict__ w, float eps,
+// grid (ceil(H / 4), M): one wave per head; the gate enters as it is, through silu or through a sigmoid (MN_GATE_ACT_*)
+template <int ACT>
+__global__ __launch_bounds__(256) void head_rms_gate_kernel(const float* __restrict__ x, int64_t ldx, const bf16_t* __restrict__ w, float eps,
                                                                  const float* __restrict__ g, int64_t ldg, float* __restrict__ y, int64_t ldy,
                                                                  bf16_t* __restrict__ y16, int64_t ldy16, int H, int vdim) {
   const int m = blockIdx.y, h = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
@@ -582,7 +517,8 @@ __global__ __launch_bounds__(256) void head_rms_silu_gate_kernel(const float* __
   for (int c = lane; c < vdim; c += 64) ss = fmaf(xr[c], xr[c], ss);
   const float den = sqrtf(wave_sum(ss) / (float)vdim + eps);
   for (int c = lane; c < vdim; c += 64) {
-    const float v = xr[c] / den * bf16_to_f32(w[c]) * silu_x(g[(int64_t)m * ldg + (int64_t)h * vdim + c]);
+    const float gv = g[(int64_t)m * ldg + (int64_t)h * vdim + c];
+    const float v = xr[c] / den * bf16_to_f32(w[c]) * (ACT == MN_GATE_ACT_SILU ? silu_x(gv) : (ACT == MN_GATE_ACT_SIGMOID ? sigmoid_f(gv) : gv));
     if (y) y[(int64_t)m * ldy + (int64_t)h * vdim + c] = v;
     if (y16) y16[(int64_t)m * ldy16 + (int64_t)h * vdim + c] = f32_to_bf16(v);
   }
@@ -652,8 +588,8 @@ extern "C" int mn_delta_prep_rows(const float* proj, int64_t ld, int M, int H, i
                                   const uint16_t* w_conv, int taps, float* state, int advance_state, const float* a_log,
                                   const float* dt_bias, float unit_eps, float q_scale, const int32_t* row_seq, const int32_t* row_slot,
                                   const int32_t* row_back, float* qkv, int64_t ldo, float* bd, int64_t ldbd, void* stream) {
-  MN_CHECK_ARG(proj && w_conv && a_log && dt_bias && row_seq && row_slot && row_back && qkv && bd && M >= 1 && H >= 1 && G >= 1 && (H % G) == 0 &&
-                   dim >= 1 && vdim >= 1 && taps >= 1 && (taps == 1 || state) && ldbd >= 2 * (int64_t)H,
+  MN_CHECK_ARG(proj && w_conv && (!a_log || dt_bias) && row_seq && row_slot && row_back && qkv && bd && M >= 1 && H >= 1 && G >= 1 && (H % G) == 0 &&
+                   dim >= 1 && vdim >= 1 && taps >= 1 && (taps == 1 || state) && ldbd >= (a_log ? 2 : 1) * (int64_t)H,
                "mn_delta_prep_rows: bad args");
   DeltaPrepArgs a{proj, ld, H, G, dim, vdim, taps, off_b, off_a, w_conv, state, advance_state ? 1 : 0, a_log, dt_bias, unit_eps, q_scale, row_seq, row_slot, row_back,
                   qkv, ldo, bd, ldbd};
@@ -700,9 +636,17 @@ extern "C" int mn_gated_delta_rows(const float* qkv, int64_t ld, const float* bd
 
 extern "C" int mn_head_rms_silu_gate_rows(const float* x, int64_t ldx, const uint16_t* w, float eps, const float* g, int64_t ldg, float* y,
                                           int64_t ldy, uint16_t* y16, int64_t ldy16, int M, int H, int vdim, void* stream) {
-  MN_CHECK_ARG(x && w && g && (y || y16) && M >= 1 && M <= 65535 && H >= 1 && vdim >= 1, "mn_head_rms_silu_gate_rows: bad args");
-  hipLaunchKernelGGL(head_rms_silu_gate_kernel, dim3((unsigned)mn_cdiv(H, 4), (unsigned)M), dim3(256), 0, mn_stream(stream), x, ldx, w, eps, g,
-                     ldg, y, ldy, y16, ldy16, H, vdim);
-  MN_CHECK_LAUNCH("mn_head_rms_silu_gate_rows");
+  return mn_head_rms_gate_rows(x, ldx, w, eps, g, ldg, MN_GATE_ACT_SILU, y, ldy, y16, ldy16, M, H, vdim, stream);
+}
+
+extern "C" int mn_head_rms_gate_rows(const float* x, int64_t ldx, const uint16_t* w, float eps, const float* g, int64_t ldg, int act, float* y,
+                                     int64_t ldy, uint16_t* y16, int64_t ldy16, int M, int H, int vdim, void* stream) {
+  MN_CHECK_ARG(x && w && g && (y || y16) && M >= 1 && M <= 65535 && H >= 1 && vdim >= 1 && act >= MN_GATE_ACT_NONE && act <= MN_GATE_ACT_SIGMOID,
+               "mn_head_rms_gate_rows: bad args");
+  const dim3 grid((unsigned)mn_cdiv(H, 4), (unsigned)M);
+#define MN_HG(A_) hipLaunchKernelGGL((head_rms_gate_kernel<A_>), grid, dim3(256), 0, mn_stream(stream), x, ldx, w, eps, g, ldg, y, ldy, y16, ldy16, H, vdim)
+  if (act == MN_GATE_ACT_SILU) MN_HG(MN_GATE_ACT_SILU); else if (act == MN_GATE_ACT_SIGMOID) MN_HG(MN_GATE_ACT_SIGMOID); else MN_HG(MN_GATE_ACT_NONE);
+#undef MN_HG
+  MN_CHECK_LAUNCH("mn_head_rms_gate_rows");
   return MN_OK;
 }

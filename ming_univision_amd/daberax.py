@@ -34,10 +34,9 @@ import os
 
 import torch
 
-from . import _lib
 from ._lib import PnLayer, PnModel, PnState, check, current_stream, lib, ptr
 from .configuration import DaberaxConfig, daberax_param_shapes
-from .seq_lm import ARITH, SeqCausalLM, SeqDecoder
+from .seq_lm import ARITH, SeqCausalLM, SeqDecoder, SequenceArenas
 
 KIND = {"attention": 0, "latent_attention": 1, "delta": 2}
 UNIT_EPS = 1e-6          # inside the root of the delta rule's unit norms: fixed by the design
@@ -54,7 +53,7 @@ def rotary_frequencies(rot, device):
     return torch.tensor(list(host), dtype=torch.float32, device=device)
 
 
-class DaberaxDecoder(SeqDecoder):
+class DaberaxDecoder(SequenceArenas, SeqDecoder):
     """Weights + per-layer caches and states + the C-ABI tables of the stack."""
 
     def __init__(self, cfg: DaberaxConfig, sd, t_max=2048, n_seq=1, arith="bf16"):
@@ -137,25 +136,13 @@ class DaberaxDecoder(SeqDecoder):
         s.layers = C.cast(layers, C.POINTER(PnLayer))
         s.final_w = self._p(sd["final.norm"])
         self.struct = s
-        self.state_t = self._alloc_state(self.n_seq)
-        self._bind_state()
+        self._init_state()
         self.block_rows = int(lib().mn_window_attn_block_rows())
         self._ws, self._decode_tabs = {}, {}
 
-    def _p(self, t):
-        assert t.dtype == torch.bfloat16 and t.is_cuda
-        t = t.contiguous()
-        self._keep.append(t)
-        return t.data_ptr()
-
-    def _f(self, t):
-        assert t.dtype == torch.float32 and t.is_cuda
-        t = t.contiguous()
-        self._keep.append(t)
-        return t.data_ptr()
-
     # ---- caches and states ---------------------------------------------------------------------------------------------------
     STATE_KEYS = ("k", "v", "conv", "lin")
+    STATE_STRUCT = PnState
     PER_TOKEN = ("k", "v")                              # arenas with one row per cached token
 
     def _state_shapes(self, n_seq):
@@ -165,45 +152,6 @@ class DaberaxDecoder(SeqDecoder):
             out.append({k: (None if d.get(k) is None else ((n_seq, self.t_max) if k in self.PER_TOKEN else (n_seq,)) + tuple(d[k]))
                         for k in self.STATE_KEYS})
         return out
-
-    def _alloc_state(self, n_seq):
-        return [{k: (None if shp is None else torch.zeros(shp, dtype=torch.float32, device=self.device)) for k, shp in ly.items()}
-                for ly in self._state_shapes(n_seq)]
-
-    def state_bytes_per_sequence(self):
-        return sum(4 * int(torch.Size(shp).numel()) for ly in self._state_shapes(1) for shp in ly.values() if shp is not None)
-
-    def _bind_state(self):
-        self._tabs = {k: _lib.ptr_array([ly[k] for ly in self.state_t]) for k in self.STATE_KEYS}
-        st = PnState()
-        for k in self.STATE_KEYS:
-            setattr(st, k, C.cast(self._tabs[k], _lib.PP))
-        st.n_seq, st.t_max = self.n_seq, self.t_max
-        self.state = st
-
-    def ensure_sequences(self, n_seq):
-        """Grow the caches and states to `n_seq` cache sequences; the existing ones keep their contents."""
-        if n_seq <= self.n_seq:
-            return
-        need = n_seq * self.state_bytes_per_sequence()
-        free, _ = torch.cuda.mem_get_info(self.device)
-        if need > free:
-            raise MemoryError(f"{n_seq} cache sequences at t_max = {self.t_max} need {need / 2**30:.1f} GiB, {free / 2**30:.1f} GiB free")
-        new = self._alloc_state(n_seq)
-        for old_ly, new_ly in zip(self.state_t, new):
-            for k, t in old_ly.items():
-                if t is not None:
-                    new_ly[k][:self.n_seq].copy_(t)
-        self.state_t, self.n_seq = new, n_seq
-        self._bind_state()
-
-    def release_sequences(self, n_keep):
-        """Shrink back to the first `n_keep` cache sequences."""
-        if n_keep >= self.n_seq:
-            return
-        self.state_t = [{k: (None if t is None else t[:n_keep].clone()) for k, t in ly.items()} for ly in self.state_t]
-        self.n_seq = n_keep
-        self._bind_state()
 
     # ---- construction ---------------------------------------------------------------------------------------------------------
     @classmethod

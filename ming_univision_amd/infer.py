@@ -43,7 +43,8 @@ def load_safetensors_dir(path):
 
 def load_model(path, dtype="bf16", device="cuda", **kw):
     """The served model of a checkpoint directory, its class chosen by config.json (configuration.MODEL_REGISTRY):
-    "pizitar" -> PizitarForCausalLM, "sakinex" -> SakinexForCausalLM, "zuzenex" -> ZuzenexForCausalLM, "daberax" -> DaberaxForCausalLM (dtype "bf16" | "f32" = the matrix-product arithmetic; kw: t_max,
+    "pizitar" -> PizitarForCausalLM, "sakinex" -> SakinexForCausalLM, "zuzenex" -> ZuzenexForCausalLM, "daberax" -> DaberaxForCausalLM,
+    "sabezen" -> SabezenForCausalLM (dtype "bf16" | "f32" = the matrix-product arithmetic; kw: t_max,
     eos_token_id),
     "ming_univision" -> MingUniVisionInfer (dtype = the weight format)."""
     from .configuration import config_from_pretrained
@@ -60,6 +61,9 @@ def load_model(path, dtype="bf16", device="cuda", **kw):
     if name == "daberax":
         from .daberax import DaberaxForCausalLM
         return DaberaxForCausalLM.from_pretrained(path, device=device, arith=dtype, **kw)
+    if name == "sabezen":
+        from .sabezen import SabezenForCausalLM
+        return SabezenForCausalLM.from_pretrained(path, device=device, arith=dtype, **kw)
     return MingUniVisionInfer(path, dtype=dtype, device=device, **kw)
 
 

@@ -1,7 +1,7 @@
 """What the decoder-only language models of this framework share: stepping rows of several cache sequences through a stack in
 passes, the vocabulary projection and the picks, a decode step captured as a HIP graph, and the lock-step generation loop.
 
-A decoder class (`pizitar.PizitarDecoder`, `sakinex.SakinexDecoder`, `zuzenex.ZuzenexDecoder`) owns its weights, caches and states and gives
+A decoder class (`pizitar.PizitarDecoder`, `sakinex.SakinexDecoder`, `zuzenex.ZuzenexDecoder`, ..) owns its weights, caches and states and gives
     step(x, row_seq, row_slot, row_back, row_len, blk_tab, max_len, out, trace, ws, distinct)   one pass over <= max_rows() rows
     _workspace_bytes(rows, max_len), ensure_sequences(n), release_sequences(n), n_trace (residual streams a trace holds)
 (a decoder with a `chunk_rows` attribute also gets chunk_tab = its rows cut into chunks of that many rows of one sequence; a decoder
@@ -13,7 +13,7 @@ import ctypes as C
 import numpy as np
 import torch
 
-from . import ops
+from . import _lib, ops
 from ._lib import check, current_stream, lib, ptr
 from .sequences import SequenceSlots, rows_of_spans
 
@@ -109,6 +109,117 @@ class SeqDecoder:
         """Sampled pick of every row at the caller's uniforms u fp32 [M] (temperature -> top-k -> top-p -> one draw)."""
         return ops.sample_logits(self.logits(hidden), u, temperature, top_k, top_p)
 
+
+
+class SequenceArenas:
+    """Caches and states of a decoder, one set of fp32 tensors per layer run with the cache sequence as the first axis.  The decoder gives
+    STATE_KEYS and STATE_STRUCT (the C-ABI table with one pointer array per key, n_seq and t_max) and `_state_shapes(n_seq)` = per run
+    {key: shape or None}, and starts with `_init_state()`.  Nothing is cleared when a sequence's number is reused."""
+
+    def _p(self, t):
+        """Device address of a packed bf16 tensor that lives as long as the decoder."""
+        assert t.dtype == torch.bfloat16 and t.is_cuda
+        t = t.contiguous()
+        self._keep.append(t)
+        return t.data_ptr()
+
+    def _f(self, t):
+        """The same for an fp32 tensor."""
+        assert t.dtype == torch.float32 and t.is_cuda
+        t = t.contiguous()
+        self._keep.append(t)
+        return t.data_ptr()
+
+    def _init_state(self):
+        self.state_t = self._alloc_state(self.n_seq)
+        self._bind_state()
+
+    def _alloc_state(self, n_seq):
+        return [{k: (None if shp is None else torch.zeros(shp, dtype=torch.float32, device=self.device)) for k, shp in run.items()}
+                for run in self._state_shapes(n_seq)]
+
+    def state_bytes_per_sequence(self):
+        return sum(4 * int(torch.Size(shp).numel()) for run in self._state_shapes(1) for shp in run.values() if shp is not None)
+
+    def _bind_state(self):
+        self._tabs = {k: _lib.ptr_array([run.get(k) for run in self.state_t]) for k in self.STATE_KEYS}
+        st = self.STATE_STRUCT()
+        for k in self.STATE_KEYS:
+            setattr(st, k, C.cast(self._tabs[k], _lib.PP))
+        st.n_seq, st.t_max = self.n_seq, self.t_max
+        self.state = st
+
+    def ensure_sequences(self, n_seq):
+        """Grow the caches and states to `n_seq` cache sequences; the existing ones keep their contents."""
+        if n_seq <= self.n_seq:
+            return
+        need = n_seq * self.state_bytes_per_sequence()
+        free, _ = torch.cuda.mem_get_info(self.device)
+        if need > free:
+            raise MemoryError(f"{n_seq} cache sequences at t_max = {self.t_max} need {need / 2**30:.1f} GiB, {free / 2**30:.1f} GiB free")
+        new = self._alloc_state(n_seq)
+        for old_run, new_run in zip(self.state_t, new):
+            for k, t in old_run.items():
+                if t is not None:
+                    new_run[k][:self.n_seq].copy_(t)
+        self.state_t, self.n_seq = new, n_seq
+        self._bind_state()
+
+    def release_sequences(self, n_keep):
+        """Shrink back to the first `n_keep` cache sequences."""
+        if n_keep >= self.n_seq:
+            return
+        self.state_t = [{k: (None if t is None else t[:n_keep].clone()) for k, t in run.items()} for run in self.state_t]
+        self.n_seq = n_keep
+        self._bind_state()
+
+
+class HybridSteps(SequenceArenas):
+    """A decoder whose passes run on the hybrid-mixer step function (mn_hyb_step): `struct` = its HybModel, `runs` = the layer of every
+    layer run, `chunk_rows` where the recurrences take chunk tables."""
+    STATE_KEYS = ("k", "v", "lin", "conv")
+    STATE_STRUCT = _lib.HybState
+
+    def _workspace_bytes(self, rows, max_len):
+        return lib().mn_hyb_workspace_bytes(C.byref(self.struct), rows)
+
+    def max_rows(self):
+        """Rows of one pass: the (row, expert) pairs of a pass are at most 65535."""
+        top = max([int(ly["mlp"]["router"]["top"]) for ly in self.cfg.layers if ly.get("mlp") and ly["mlp"]["kind"] == "moe"] or [1])
+        return max(1, min(MAX_ROWS, 65535 // top))
+
+    def step(self, x, row_seq, row_slot, row_back, row_len=None, blk_tab=None, max_len=None, out=None, trace=None, ws=None, distinct=False,
+             chunk_tab=None, row_tok=None):
+        """One pass of the stack over M rows.  x fp32 [M, width] (input embeddings); int32 device arrays per row (row r is position
+        row_slot[r] of cache sequence row_seq[r], preceded in this pass by row_back[r] rows of its sequence, and token row_tok[r] where
+        the layers read ids); blk_tab int32 [n_blk, 2] cuts the rows into runs of <= block_rows consecutive rows of one sequence (not
+        read when distinct) and chunk_tab int32 [n_chunks, 2] into chunks of <= chunk_rows (optional: without it the recurrences walk
+        their rows one by one); row_len is the other decoder's table and is not read here; max_len (host int) >= every position + 1
+        (default: the cache's length).  Appends the rows' keys and values and advances the filter and recurrent states.  trace: optional
+        fp32 [runs, M, width] that receives the residual stream after every layer run.  distinct: every row is alone in its sequence (a
+        decode step).  Returns the final norm's output [M, width] fp32."""
+        M = x.shape[0]
+        assert x.dtype == torch.float32 and x.is_cuda and x.stride(1) == 1 and x.shape[1] == self.cfg.width and 1 <= M <= self.max_rows()
+        for t in (row_seq, row_slot, row_back) + ((row_tok,) if self.needs_tokens else ()):
+            assert t is not None and t.dtype == torch.int32 and t.is_cuda and t.is_contiguous() and t.numel() >= M
+        max_len = self.t_max if max_len is None else int(max_len)
+        assert 1 <= max_len <= self.t_max, f"{max_len} tokens exceed the cache (t_max = {self.t_max})"
+        if not distinct:
+            assert blk_tab is not None and blk_tab.dtype == torch.int32 and blk_tab.is_cuda and blk_tab.is_contiguous() and blk_tab.shape[1] == 2
+        if chunk_tab is not None:
+            assert chunk_tab.dtype == torch.int32 and chunk_tab.is_cuda and chunk_tab.is_contiguous() and chunk_tab.shape[1] == 2
+        if out is None:
+            out = torch.empty(M, self.cfg.width, dtype=torch.float32, device=self.device)
+        if trace is not None:
+            assert trace.dtype == torch.float32 and trace.is_contiguous() and tuple(trace.shape) == (self.n_trace, M, self.cfg.width)
+        if ws is None:
+            ws = self._workspace(M, max_len)
+        use_chunks = chunk_tab is not None and not distinct
+        check(lib().mn_hyb_step(C.byref(self.struct), C.byref(self.state), ptr(x), x.stride(0), M, ptr(row_tok), ptr(row_seq), ptr(row_slot),
+                                ptr(row_back), None if distinct else ptr(blk_tab), M if distinct else blk_tab.shape[0],
+                                ptr(chunk_tab) if use_chunks else None, chunk_tab.shape[0] if use_chunks else 0, max_len,
+                                1 if distinct else 0, ptr(out), ptr(trace), ptr(ws), ws.numel(), current_stream()), "mn_hyb_step")
+        return out
 
 
 class DecodeGraph:

@@ -32,16 +32,15 @@ import os
 
 import torch
 
-from . import _lib
-from ._lib import HybLayer, HybModel, HybState, check, current_stream, lib, ptr
+from ._lib import HybLayer, HybModel, lib
 from .configuration import ZuzenexConfig, zuzenex_param_shapes
-from .seq_lm import ARITH, SeqCausalLM, SeqDecoder
+from .seq_lm import ARITH, HybridSteps, SeqCausalLM, SeqDecoder
 
 KIND = {"attention": 0, "lightning": 1}
 FF_NONE, FF_DENSE, FF_MOE = 0, 1, 2
 
 
-class ZuzenexDecoder(SeqDecoder):
+class ZuzenexDecoder(HybridSteps, SeqDecoder):
     """Weights + per-run caches and states + the C-ABI tables of the stack."""
 
     def __init__(self, cfg: ZuzenexConfig, sd, t_max=2048, n_seq=1, arith="bf16"):
@@ -113,27 +112,12 @@ class ZuzenexDecoder(SeqDecoder):
         s.run_layer = self._run_layer
         s.final_w = self._p(sd["final.norm"])
         self.struct = s
-        self.state_t = self._alloc_state(self.n_seq)
-        self._bind_state()
         self.block_rows = int(lib().mn_window_attn_block_rows())
         self.chunk_rows = int(lib().mn_lightning_chunk_rows())
+        self._init_state()
         self._ws, self._decode_tabs = {}, {}
 
-    def _p(self, t):
-        assert t.dtype == torch.bfloat16 and t.is_cuda
-        t = t.contiguous()
-        self._keep.append(t)
-        return t.data_ptr()
-
-    def _f(self, t):
-        assert t.dtype == torch.float32 and t.is_cuda
-        t = t.contiguous()
-        self._keep.append(t)
-        return t.data_ptr()
-
     # ---- caches and states ---------------------------------------------------------------------------------------------------
-    STATE_KEYS = ("k", "v", "lin")
-
     def _state_shapes(self, n_seq):
         """Per run: {name: shape or None}."""
         out = []
@@ -143,45 +127,6 @@ class ZuzenexDecoder(SeqDecoder):
             out.append({"k": (n_seq, self.t_max, ck) if attn else None, "v": (n_seq, self.t_max, cv) if attn else None,
                         "lin": None if attn else (n_seq, H, d, e)})
         return out
-
-    def _alloc_state(self, n_seq):
-        return [{k: (None if shp is None else torch.zeros(shp, dtype=torch.float32, device=self.device)) for k, shp in run.items()}
-                for run in self._state_shapes(n_seq)]
-
-    def state_bytes_per_sequence(self):
-        return sum(4 * int(torch.Size(shp).numel()) for run in self._state_shapes(1) for shp in run.values() if shp is not None)
-
-    def _bind_state(self):
-        self._tabs = {k: _lib.ptr_array([run[k] for run in self.state_t]) for k in self.STATE_KEYS}
-        st = HybState()
-        for k in self.STATE_KEYS:
-            setattr(st, k, C.cast(self._tabs[k], _lib.PP))
-        st.n_seq, st.t_max = self.n_seq, self.t_max
-        self.state = st
-
-    def ensure_sequences(self, n_seq):
-        """Grow the caches and states to `n_seq` cache sequences; the existing ones keep their contents."""
-        if n_seq <= self.n_seq:
-            return
-        need = n_seq * self.state_bytes_per_sequence()
-        free, _ = torch.cuda.mem_get_info(self.device)
-        if need > free:
-            raise MemoryError(f"{n_seq} cache sequences at t_max = {self.t_max} need {need / 2**30:.1f} GiB, {free / 2**30:.1f} GiB free")
-        new = self._alloc_state(n_seq)
-        for old_run, new_run in zip(self.state_t, new):
-            for k, t in old_run.items():
-                if t is not None:
-                    new_run[k][:self.n_seq].copy_(t)
-        self.state_t, self.n_seq = new, n_seq
-        self._bind_state()
-
-    def release_sequences(self, n_keep):
-        """Shrink back to the first `n_keep` cache sequences."""
-        if n_keep >= self.n_seq:
-            return
-        self.state_t = [{k: (None if t is None else t[:n_keep].clone()) for k, t in run.items()} for run in self.state_t]
-        self.n_seq = n_keep
-        self._bind_state()
 
     # ---- construction ---------------------------------------------------------------------------------------------------------
     @classmethod
@@ -211,48 +156,6 @@ class ZuzenexDecoder(SeqDecoder):
             else:
                 sd[k] = synth_tensor(k, shp, seed, device, torch.bfloat16, mean=0.0, std=shp[-1] ** -0.5)
         return cls(cfg, sd, **kw)
-
-    # ---- stepping -------------------------------------------------------------------------------------------------------------
-    def _workspace_bytes(self, rows, max_len):
-        return lib().mn_hyb_workspace_bytes(C.byref(self.struct), rows)
-
-    def max_rows(self):
-        """Rows of one pass: the (row, expert) pairs of a pass are at most 65535."""
-        top = max([int(ly["mlp"]["router"]["top"]) for ly in self.cfg.layers if ly.get("mlp") and ly["mlp"]["kind"] == "moe"] or [1])
-        return max(1, min(super().max_rows(), 65535 // top))
-
-    def step(self, x, row_seq, row_slot, row_back, row_len=None, blk_tab=None, max_len=None, out=None, trace=None, ws=None, distinct=False,
-             chunk_tab=None):
-        """One pass of the stack over M rows.  x fp32 [M, width] (input embeddings); int32 device arrays per row (row r is position
-        row_slot[r] of cache sequence row_seq[r], preceded in this pass by row_back[r] rows of its sequence); blk_tab int32 [n_blk, 2]
-        cuts the rows into runs of <= block_rows consecutive rows of one sequence (not read when distinct) and chunk_tab int32
-        [n_chunks, 2] into chunks of <= chunk_rows (optional: without it the recurrences walk their rows one by one); row_len is the
-        other decoder's table and is not read here; max_len (host int) >= every position + 1 (default: the cache's length).  Appends
-        the rows' keys and values and advances the recurrent states.  trace: optional fp32 [runs, M, width] that receives the
-        residual stream after every layer run.  distinct: every row is alone in its sequence (a decode step).  Returns the final
-        norm's output [M, width] fp32."""
-        M = x.shape[0]
-        assert x.dtype == torch.float32 and x.is_cuda and x.stride(1) == 1 and x.shape[1] == self.cfg.width and 1 <= M <= self.max_rows()
-        for t in (row_seq, row_slot, row_back):
-            assert t.dtype == torch.int32 and t.is_cuda and t.is_contiguous() and t.numel() >= M
-        max_len = self.t_max if max_len is None else int(max_len)
-        assert 1 <= max_len <= self.t_max, f"{max_len} tokens exceed the cache (t_max = {self.t_max})"
-        if not distinct:
-            assert blk_tab is not None and blk_tab.dtype == torch.int32 and blk_tab.is_cuda and blk_tab.is_contiguous() and blk_tab.shape[1] == 2
-        if chunk_tab is not None:
-            assert chunk_tab.dtype == torch.int32 and chunk_tab.is_cuda and chunk_tab.is_contiguous() and chunk_tab.shape[1] == 2
-        if out is None:
-            out = torch.empty(M, self.cfg.width, dtype=torch.float32, device=self.device)
-        if trace is not None:
-            assert trace.dtype == torch.float32 and trace.is_contiguous() and tuple(trace.shape) == (self.n_trace, M, self.cfg.width)
-        if ws is None:
-            ws = self._workspace(M, max_len)
-        use_chunks = chunk_tab is not None and not distinct
-        check(lib().mn_hyb_step(C.byref(self.struct), C.byref(self.state), ptr(x), x.stride(0), M, ptr(row_seq), ptr(row_slot), ptr(row_back),
-                                None if distinct else ptr(blk_tab), M if distinct else blk_tab.shape[0],
-                                ptr(chunk_tab) if use_chunks else None, chunk_tab.shape[0] if use_chunks else 0, max_len,
-                                1 if distinct else 0, ptr(out), ptr(trace), ptr(ws), ws.numel(), current_stream()), "mn_hyb_step")
-        return out
 
 
 class ZuzenexForCausalLM(SeqCausalLM):
