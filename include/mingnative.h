@@ -1171,7 +1171,7 @@ MN_API size_t mn_sizeof_hyb_model(void);
 MN_API size_t mn_sizeof_hyb_state(void);
 /* One pass of the stack over M rows; rows, row arrays, blk_tab / n_blk, max_len, flags, out and trace as mn_pmix_step (trace: fp32
  * [n_runs, M, width]).  chunk_tab / n_chunks: the rows cut into chunks of <= mn_lightning_chunk_rows() consecutive rows of one
- * sequence (NULL / 0: the recurrences walk their rows one by one).  row_tok int32 [M]: the rows' token ids (read by layers with a table). */
+ * sequence (for stacks with gla layers: <= mn_channel_chunk_rows(); NULL / 0: the recurrences walk their rows one by one).  row_tok int32 [M]: the rows' token ids (read by layers with a table). */
 MN_API size_t mn_hyb_workspace_bytes(const mn_hyb_model* m, int M);
 MN_API int mn_hyb_step(const mn_hyb_model* m, const mn_hyb_state* st, const float* x, int64_t ldx, int M, const int32_t* row_tok,
                        const int32_t* row_seq, const int32_t* row_slot, const int32_t* row_back, const int32_t* blk_tab, int n_blk,
@@ -1339,6 +1339,30 @@ typedef struct mn_low_rank_job {
   float root;
 } mn_low_rank_job;
 MN_API int mn_low_rank_gate_rows(const mn_low_rank_job* jobs, int n_jobs, int M, void* stream);
+/* What the rows of a decode step (every row alone in its sequence, M <= 64) compute between a layer's stacked product and its recurrence, in
+ * ONE launch; every part is optional: the delta rule's preparation as mn_delta_prep_rows with the state moved on (delta != 0), up to two
+ * low-rank jobs, xIELU (act_n > 0), table rows by token id (top > 0). */
+typedef struct mn_rows_prep {
+  const float* proj; int64_t ld;                   /* delta: raw [q ; k ; v] at column 0, write-strength logits at off_b */
+  int32_t delta, H, G, dim, vdim, taps, off_b;
+  const uint16_t* w_conv;
+  float* conv_state;
+  float unit_eps, q_scale;
+  float* qkv; int64_t ldqkv;
+  float* beta; int64_t ldbeta;
+  int32_t n_jobs;
+  mn_low_rank_job job[2];
+  const float* act_x; int64_t ld_act_x;
+  float act_pos, act_neg;
+  float* act_y; int64_t ld_act_y;
+  int32_t act_n;
+  const int32_t *table, *tok;
+  int32_t vocab, top;
+  int32_t* idx;
+} mn_rows_prep;
+MN_API size_t mn_sizeof_low_rank_job(void);
+MN_API size_t mn_sizeof_rows_prep(void);
+MN_API int mn_rows_prep_launch(const mn_rows_prep* a, const int32_t* row_seq, const int32_t* row_slot, int M, void* stream);
 /* Recurrence with a decay per key channel over each sequence's rows, per head h (q / k head h / (H / G)): S <- diag(g) S with g = the row's
  * dim decays of the head (g fp32 [M, H dim]); then with beta (fp32 [M, H]) the delta rule's write u = beta (v - S^T k), S <- S + k u^T,
  * with beta NULL the plain write S <- S + k v^T; out[m, h vdim + c] = o_scale (S^T q)[c].  qkv fp32 [M, ld] = [q: G dim ; k: G dim ; v: H
@@ -1348,6 +1372,15 @@ MN_API int mn_low_rank_gate_rows(const mn_low_rank_job* jobs, int n_jobs, int M,
 MN_API int mn_channel_state_rows(const float* qkv, int64_t ld, const float* g, int64_t ldg, const float* beta, int64_t ldb, int M, int H, int G,
                                  int dim, int vdim, float o_scale, float* state, const int32_t* row_seq, const int32_t* row_slot,
                                  const int32_t* row_back, const int32_t* blk_tab, int n_blk, int flags, float* out, int64_t ldo, void* stream);
+/* The plain write as a chunked scan, for steps of many rows: chunks of <= mn_channel_chunk_rows() rows of one sequence (chunk_tab int32
+ * [n_chunks, 2] = (first row, rows), in row order); every chunk's end state from zero and its decay product per key channel, the start
+ * states carried along each sequence, every chunk's outputs from its start state.  dim <= 256. */
+MN_API int mn_channel_chunk_rows(void);
+MN_API size_t mn_channel_scan_workspace_bytes(int n_chunks, int H, int dim, int vdim);
+MN_API int mn_channel_state_rows_scan(const float* qkv, int64_t ld, const float* g, int64_t ldg, int M, int H, int G, int dim, int vdim,
+                                      float o_scale, float* state, const int32_t* row_seq, const int32_t* row_slot, const int32_t* row_back,
+                                      const int32_t* chunk_tab, int n_chunks, float* out, int64_t ldo, void* workspace, size_t workspace_bytes,
+                                      void* stream);
 /* mn_head_rms_silu_gate_rows with the gate's function named: the gate as it is, through silu, or through a sigmoid */
 enum { MN_GATE_ACT_NONE = 0, MN_GATE_ACT_SILU = 1, MN_GATE_ACT_SIGMOID = 2 };
 MN_API int mn_head_rms_gate_rows(const float* x, int64_t ldx, const uint16_t* w, float eps, const float* g, int64_t ldg, int act, float* y,
@@ -1359,7 +1392,7 @@ MN_API int mn_gemv_glu_indexed(const float* A, int64_t lda, int a_div, const uin
  * fp32 [H, H]) over the keys j of the row's sequence with j <= pos, pos - j < window (window > 0) and floor(j / chunk) = floor(pos / chunk)
  * (chunk > 0), softmax with exp(sink[h]) added to the denominator (sink DEVICE fp32 [H] or NULL), values of key/value head h / (H / G)
  * with dim values; arenas [n_seq, t_max, ld].  blk_tab int32 [n_blk, 2]: runs of <= rows consecutive rows of one sequence (NULL: every
- * row is a run, rows = 1, n_blk = M).  rows: at most mn_talk_attn_block_rows(H, G, dim) for the matrix-core kernel (0: no instance; the
+ * row is a run, rows = 1, n_blk = M).  rows: at most mn_talk_attn_block_rows(H, G, dim) for the matrix-core kernel (dim % 4 == 0, 16-byte aligned rows; 0: no instance; the
  * plain kernel takes H <= 112, H dim <= 16384).  nsplit key splits (mn_talk_attn_splits proposes) with a workspace and a merge launch.
  * variant -1: the matrix-core kernel where it has an instance. */
 enum { MN_TALK_ATTN_MFMA = 0, MN_TALK_ATTN_PLAIN = 1 };

@@ -165,6 +165,15 @@ class LowRankJob(C.Structure):
                 ("ldo", C.c_int64), ("k", C.c_int32), ("n", C.c_int32), ("kind", C.c_int32), ("head_n", C.c_int32), ("root", C.c_float)]
 
 
+class RowsPrep(C.Structure):
+    _fields_ = [("proj", C.c_void_p), ("ld", C.c_int64)] + [(k, C.c_int32) for k in ("delta", "H", "G", "dim", "vdim", "taps", "off_b")] + \
+               [("w_conv", C.c_void_p), ("conv_state", C.c_void_p), ("unit_eps", C.c_float), ("q_scale", C.c_float), ("qkv", C.c_void_p),
+                ("ldqkv", C.c_int64), ("beta", C.c_void_p), ("ldbeta", C.c_int64), ("n_jobs", C.c_int32), ("job", LowRankJob * 2),
+                ("act_x", C.c_void_p), ("ld_act_x", C.c_int64), ("act_pos", C.c_float), ("act_neg", C.c_float), ("act_y", C.c_void_p),
+                ("ld_act_y", C.c_int64), ("act_n", C.c_int32), ("table", C.c_void_p), ("tok", C.c_void_p), ("vocab", C.c_int32),
+                ("top", C.c_int32), ("idx", C.c_void_p)]
+
+
 class PnLayer(C.Structure):
     _fields_ = [(k, C.c_int32) for k in ("kind", "heads", "kv_heads", "dim", "vdim", "rot", "kv_rank", "rot_dims", "rot_interleaved", "window",
                                          "conv", "ff", "side", "has_gate")] + \
@@ -189,7 +198,8 @@ STRUCTS = ((0, "mn_sizeof_skinny_args", SkinnyArgs), (1, "mn_sizeof_rf_head", Rf
            (6, "mn_sizeof_seq_layer", SeqLayer), (7, "mn_sizeof_seq_model", SeqModel), (8, "mn_sizeof_seq_state", SeqState),
            (9, "mn_sizeof_pmix_layer", PmixLayer), (10, "mn_sizeof_pmix_model", PmixModel), (11, "mn_sizeof_pmix_state", PmixState),
            (12, "mn_sizeof_hyb_layer", HybLayer), (13, "mn_sizeof_hyb_model", HybModel), (14, "mn_sizeof_hyb_state", HybState),
-           (15, "mn_sizeof_pn_layer", PnLayer), (16, "mn_sizeof_pn_model", PnModel), (17, "mn_sizeof_pn_state", PnState))
+           (15, "mn_sizeof_pn_layer", PnLayer), (16, "mn_sizeof_pn_model", PnModel), (17, "mn_sizeof_pn_state", PnState),
+           (18, "mn_sizeof_low_rank_job", LowRankJob), (19, "mn_sizeof_rows_prep", RowsPrep))
 
 
 def check_struct_layouts(handle):
@@ -417,8 +427,13 @@ SYMBOLS = {
     "mn_add_layernorm_rows": (_i, [_p, _i64, _p, _i64, _p, _i64, _p, _p, _f, _i, _p, _f, _p, _i64, _p, _i64, _i, _i, _p]),
     "mn_xielu_rows": (_i, [_p, _i64, _f, _f, _p, _i64, _p, _i64, _i, _i, _p]),
     "mn_token_table_rows": (_i, [_p, _i, _i, _p, _i, _p, _p, _p]),
+    "mn_sizeof_low_rank_job": (_sz, []), "mn_sizeof_rows_prep": (_sz, []),
+    "mn_rows_prep_launch": (_i, [C.POINTER(RowsPrep), _p, _p, _i, _p]),
     "mn_low_rank_gate_rows": (_i, [C.POINTER(LowRankJob), _i, _i, _p]),
     "mn_channel_state_rows": (_i, [_p, _i64, _p, _i64, _p, _i64, _i, _i, _i, _i, _i, _f, _p, _p, _p, _p, _p, _i, _i, _p, _i64, _p]),
+    "mn_channel_chunk_rows": (_i, []),
+    "mn_channel_scan_workspace_bytes": (_sz, [_i, _i, _i, _i]),
+    "mn_channel_state_rows_scan": (_i, [_p, _i64, _p, _i64, _i, _i, _i, _i, _i, _f, _p, _p, _p, _p, _p, _i, _p, _i64, _p, _sz, _p]),
     "mn_head_rms_gate_rows": (_i, [_p, _i64, _p, _f, _p, _i64, _i, _p, _i64, _p, _i64, _i, _i, _i, _p]),
     "mn_gemv_glu_indexed": (_i, [_p, _i64, _i, _p, _i64, _i64, _p, _i, _p, _i64, _i, _i, _i, _p]),
     "mn_talk_attn_block_rows": (_i, [_i, _i, _i]),

@@ -181,8 +181,19 @@ extern "C" int mn_struct_layout(int which, size_t* offsets, int cap) {
       F(k) F(v) F(conv) F(lin) F(n_seq) F(t_max)
 #undef F
   };
+  static const size_t low_rank[] = {
+#define F(f) MN_OFF(mn_low_rank_job, f)
+      F(a) F(lda) F(w) F(bias) F(a_log) F(out) F(ldo) F(k) F(n) F(kind) F(head_n) F(root)
+#undef F
+  };
+  static const size_t rows_prep[] = {
+#define F(f) MN_OFF(mn_rows_prep, f)
+      F(proj) F(ld) F(delta) F(H) F(G) F(dim) F(vdim) F(taps) F(off_b) F(w_conv) F(conv_state) F(unit_eps) F(q_scale) F(qkv) F(ldqkv) F(beta)
+      F(ldbeta) F(n_jobs) F(job) F(act_x) F(ld_act_x) F(act_pos) F(act_neg) F(act_y) F(ld_act_y) F(act_n) F(table) F(tok) F(vocab) F(top) F(idx)
+#undef F
+  };
   const size_t* tab[] = {skinny, rf, llm, semdec, comm, llm_tp, seq_layer, seq_model, seq_state, pmix_layer, pmix_model, pmix_state,
-                         hyb_layer, hyb_model, hyb_state, pn_layer, pn_model, pn_state};
+                         hyb_layer, hyb_model, hyb_state, pn_layer, pn_model, pn_state, low_rank, rows_prep};
   const int cnt[] = {(int)(sizeof(skinny) / sizeof(size_t)), (int)(sizeof(rf) / sizeof(size_t)), (int)(sizeof(llm) / sizeof(size_t)),
                      (int)(sizeof(semdec) / sizeof(size_t)), (int)(sizeof(comm) / sizeof(size_t)), (int)(sizeof(llm_tp) / sizeof(size_t)),
                      (int)(sizeof(seq_layer) / sizeof(size_t)), (int)(sizeof(seq_model) / sizeof(size_t)),
@@ -190,8 +201,9 @@ extern "C" int mn_struct_layout(int which, size_t* offsets, int cap) {
                      (int)(sizeof(pmix_model) / sizeof(size_t)), (int)(sizeof(pmix_state) / sizeof(size_t)),
                      (int)(sizeof(hyb_layer) / sizeof(size_t)), (int)(sizeof(hyb_model) / sizeof(size_t)),
                      (int)(sizeof(hyb_state) / sizeof(size_t)), (int)(sizeof(pn_layer) / sizeof(size_t)),
-                     (int)(sizeof(pn_model) / sizeof(size_t)), (int)(sizeof(pn_state) / sizeof(size_t))};
-  MN_CHECK_ARG(which >= 0 && which < 18, "mn_struct_layout: unknown struct id");
+                     (int)(sizeof(pn_model) / sizeof(size_t)), (int)(sizeof(pn_state) / sizeof(size_t)),
+                     (int)(sizeof(low_rank) / sizeof(size_t)), (int)(sizeof(rows_prep) / sizeof(size_t))};
+  MN_CHECK_ARG(which >= 0 && which < 20, "mn_struct_layout: unknown struct id");
   for (int i = 0; i < cnt[which] && i < cap; ++i) offsets[i] = tab[which][i];
   return cnt[which];
 }

@@ -4,6 +4,7 @@
 //   mn_xielu_rows             the two-sided quadratic / exponential activation
 //   mn_token_table_rows       table rows chosen by token id (the experts of a table-routed mixture)
 //   mn_low_rank_gate_rows     second stage of low-rank projections with the gate functions behind them
+//   mn_rows_prep_launch       decode rows: the delta rule's preparation, the low-rank gates, the activation and the table rows in one launch
 //   mn_channel_state_rows     S <- diag(g) S, then a delta-rule write or a plain k v^T, o = S^T q: prompt rows and decode rows
 //   mn_gemv_glu_indexed       silu(gate) * up of the expert an index names
 #include <math.h>
@@ -261,6 +262,36 @@ __device__ __forceinline__ void low_rank_few(const LowRankArgs& a, int bx, int b
 
 __global__ __launch_bounds__(256) void low_rank_few_kernel(LowRankArgs a) { low_rank_few(a, blockIdx.x, blockIdx.y, threadIdx.x); }
 
+// Decode rows: everything between the stacked product and the recurrence.  blockIdx.x runs over the parts (delta units | low-rank outputs |
+// activation | table), blockIdx.y over the rows (low-rank: over groups of LR_ROWS rows).
+struct RowsPrepArgs {
+  DeltaPrepArgs delta;
+  LowRankArgs lr;
+  XieluArgs act;
+  const int32_t *table, *tok; int vocab, top; int32_t* idx;
+  int M, n_delta, n_lr, n_act;                 // workgroups of the first three parts
+};
+__global__ __launch_bounds__(256) void rows_prep_kernel(RowsPrepArgs a) {
+  const int m = blockIdx.y, tid = threadIdx.x;
+  int b = blockIdx.x;
+  if (b < a.n_delta) {
+    delta_prep_unit(a.delta, m, b * 4 + (tid >> 6), tid & 63, 0);
+    if (b == 0) delta_prep_strengths(a.delta, m, tid);
+    return;
+  }
+  b -= a.n_delta;
+  if (b < a.n_lr) {
+    if (m * LR_ROWS < a.M) low_rank_few(a.lr, b, m, tid);
+    return;
+  }
+  b -= a.n_lr;
+  if (b < a.n_act) {
+    xielu_block(a.act, m, b, tid);
+    return;
+  }
+  for (int j = tid; j < a.top; j += 256) a.idx[m * a.top + j] = a.table[(int64_t)min(max(a.tok[m], 0), a.vocab - 1) * a.top + j];
+}
+
 // Many rows: 64 x 64 output tiles on the fp32 matrix cores (v_mfma_f32_16x16x4_f32; operand layouts in mfma_f32_tiles.h), k in pieces
 // of 32 staged as fp32; wave w owns 16 rows x 64 columns.
 __global__ __launch_bounds__(256) void low_rank_mfma_kernel(LowRankArgs a) {
@@ -315,6 +346,7 @@ struct ChanArgs {
   const int32_t* blk_tab;                    // optional: runs of rows; a sequence's first row in the call starts a run
   float* out; int64_t ldo;                   // [M, H vdim]
   int M;
+  const int32_t* chunk_tab; float* ws; float* wsp;      // scan: chunks of rows; [n_chunks, H, dim, vdim] states; [n_chunks, H, dim] decay products
 };
 
 template <int LPC>
@@ -323,30 +355,44 @@ __device__ __forceinline__ float lanes_sum(float v) { return LPC == 16 ? row16_s
 // Prompt rows, heads of at most NS LPC state rows: the workgroup of a sequence's FIRST row in the call walks that sequence's rows.  LPC
 // lanes share C neighbouring value columns (NT / LPC * C columns a workgroup); a lane holds the state rows 4 (s + LPC jj) + t, t < 4,
 // jj < NS / 4, in registers.  Rows come in batches of DBT: a batch's q, k, g, v and write strengths go global -> registers (while the
-// previous batch is computed) -> LDS; the steps then run from LDS and registers alone, the operands of step r + 1 read ahead of step r,
-// without a barrier or a memory access between steps.  LDS rows are padded with zeros to DP values, under which padded state rows stay 0.
-template <int NS, int LPC, int C, int NT, int DBT, bool DELTA>
+// previous batch is computed) -> LDS; the steps then run from LDS and registers alone, the operands of step r + 1 requested ahead of
+// step r, without a barrier or a memory access between steps.  Only the sum that the write needs (s . k) is reduced within a step; the
+// read-outs' partial sums s . q go to LDS lane by lane and are added up once per batch.  LDS rows are padded with zeros to DP values,
+// under which padded state rows stay 0.
+//   MODE WALK       from the sequence's state to its state
+//   MODE CHUNK_END  a workgroup per CHUNK of rows: from zero, no outputs; the chunk's end state and its decay product per key channel
+//   MODE CHUNK_OUT  a workgroup per chunk: from the chunk's start state in the workspace, outputs only
+enum { WALK = 0, CHUNK_END = 1, CHUNK_OUT = 2 };
+template <int NS, int LPC, int C, int NT, int DBT, bool DELTA, bool VEC, int MODE>
 __global__ __launch_bounds__(NT) void chan_walk_kernel(ChanArgs a) {
-  constexpr int CPB = NT / LPC * C, DP = NS * LPC, Q4 = DBT * DP / 4 / NT, NV = (DBT * CPB + NT - 1) / NT;
-  static_assert(Q4 * 4 * NT == DBT * DP && 2 * DBT <= NT, "a batch is staged by whole 16-byte pieces per thread");
+  constexpr int CPB = NT / LPC * C, DP = NS * LPC, Q4 = DBT * DP / 4 / NT, NV = (DBT * CPB + NT - 1) / NT, PS = LPC + 4, NP = (DP + NT - 1) / NT;
+  constexpr bool OUT = MODE != CHUNK_END;
+  static_assert(Q4 * 4 * NT == DBT * DP && DBT <= NT && DBT % 2 == 0, "a batch is staged by whole 16-byte pieces per thread");
+  static_assert(!DELTA || MODE == WALK, "the delta rule's write needs the state before it");
   __shared__ __align__(16) float opl[3][DBT][DP];             // q, k, g
   __shared__ __align__(16) float vs[DBT][CPB];
-  __shared__ __align__(16) float os[DBT][CPB];
+  __shared__ __align__(16) float part[OUT ? DBT * CPB * PS : 4];   // s . q by lanes
+  __shared__ float us[DELTA ? DBT : 1][CPB];                  // what each step wrote
   __shared__ float bs[2][DBT];                                // beta, k . q
-  const int m0 = a.blk_tab ? a.blk_tab[2 * blockIdx.y] : blockIdx.y;
-  if (a.row_back[m0] != 0) return;
+  const int m0 = MODE != WALK ? a.chunk_tab[2 * blockIdx.y] : (a.blk_tab ? a.blk_tab[2 * blockIdx.y] : blockIdx.y);
+  if (MODE == WALK && a.row_back[m0] != 0) return;
   const int ncb = (a.vdim + CPB - 1) / CPB, h = blockIdx.x / ncb, cb = blockIdx.x - h * ncb;
   const int tid = threadIdx.x, s = tid % LPC, cl = tid / LPC, c = cb * CPB + C * cl;
   const int d = a.dim, kvh = h / (a.H / a.G);
   int n = 1;
-  for (;;) {
-    const int m = m0 + n + tid;
-    const int cnt = __syncthreads_count(m < a.M && a.row_back[m] == m - m0);
-    n += cnt;
-    if (cnt < NT) break;
+  if (MODE == WALK) {
+    for (;;) {
+      const int m = m0 + n + tid;
+      const int cnt = __syncthreads_count(m < a.M && a.row_back[m] == m - m0);
+      n += cnt;
+      if (cnt < NT) break;
+    }
+  } else {
+    n = a.chunk_tab[2 * blockIdx.y + 1];
   }
-  float* sp = a.state + (((int64_t)a.row_seq[m0] * a.H + h) * d) * a.vdim;
-  const bool fresh = a.row_slot[m0] == 0;
+  const int64_t hde = (int64_t)d * a.vdim;
+  float* sp = MODE == WALK ? a.state + ((int64_t)a.row_seq[m0] * a.H + h) * hde : a.ws + ((int64_t)blockIdx.y * a.H + h) * hde;
+  const bool fresh = MODE == CHUNK_END || (MODE == WALK && a.row_slot[m0] == 0);
   float S[C][NS];
 #pragma unroll
   for (int cc = 0; cc < C; ++cc)
@@ -355,46 +401,55 @@ __global__ __launch_bounds__(NT) void chan_walk_kernel(ChanArgs a) {
       const int i = 4 * (s + LPC * (j >> 2)) + (j & 3);
       S[cc][j] = (c + cc < a.vdim && !fresh && i < d) ? sp[(int64_t)i * a.vdim + c + cc] : 0.f;
     }
-  const bool vec = (d & 3) == 0 && (a.ld & 3) == 0 && (a.ldg & 3) == 0 && (((uintptr_t)a.qkv | (uintptr_t)a.g) & 15) == 0;
+  __syncthreads();                             // the state has arrived: from here on only a batch's loads are in flight
+  float gp[NP];
+#pragma unroll
+  for (int t = 0; t < NP; ++t) gp[t] = 1.f;
   f32x4 rq[3][Q4];
   float rv[NV], rb = 0.f;
+  const float* const src0[3] = {a.qkv + (int64_t)kvh * d, a.qkv + (int64_t)(a.G + kvh) * d, a.g + (int64_t)h * d};
+  const int64_t lds_[3] = {a.ld, a.ld, a.ldg};
+  const float* const srcv = a.qkv + (int64_t)2 * a.G * d + (int64_t)h * a.vdim;
+  // raw loads at clamped addresses; what does not count is replaced when the batch goes to LDS
   auto fetch = [&](int b0) {
-    const int rows = min(DBT, n - b0);
 #pragma unroll
     for (int t = 0; t < Q4; ++t) {
       const int e = tid + NT * t, r = e / (DP / 4), i = 4 * (e % (DP / 4));
-      const int64_t m = m0 + b0 + min(r, rows - 1);
-      const float* src[3] = {a.qkv + m * a.ld + (int64_t)kvh * d, a.qkv + m * a.ld + (int64_t)(a.G + kvh) * d, a.g + m * a.ldg + (int64_t)h * d};
+      const int64_t m = m0 + min(b0 + r, n - 1);
 #pragma unroll
-      for (int w = 0; w < 3; ++w) {
-        if (vec) {
-          const f32x4 v = *reinterpret_cast<const f32x4*>(src[w] + (i < d ? i : 0));
-          rq[w][t] = (r < rows && i < d) ? v : f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int w = OUT ? 0 : 1; w < 3; ++w) {
+        const float* src = src0[w] + m * lds_[w];
+        if constexpr (VEC) {
+          rq[w][t] = *reinterpret_cast<const f32x4*>(src + min(i, d - 4));
         } else {
 #pragma unroll
-          for (int u = 0; u < 4; ++u) {
-            const float v = src[w][i + u < d ? i + u : 0];
-            rq[w][t][u] = (r < rows && i + u < d) ? v : 0.f;
-          }
+          for (int u = 0; u < 4; ++u) rq[w][t][u] = src[min(i + u, d - 1)];
         }
       }
     }
 #pragma unroll
     for (int t = 0; t < NV; ++t) {
       const int e = tid + NT * t, r = e / CPB, cc = cb * CPB + e % CPB;
-      rv[t] = (r < rows && cc < a.vdim) ? a.qkv[(int64_t)(m0 + b0 + r) * a.ld + (int64_t)2 * a.G * d + (int64_t)h * a.vdim + cc] : 0.f;
+      rv[t] = srcv[(m0 + min(b0 + r, n - 1)) * a.ld + min(cc, a.vdim - 1)];
     }
-    if (DELTA && tid < DBT) rb = tid < rows ? a.beta[(int64_t)(m0 + b0 + tid) * a.ldb + h] : 0.f;
+    if (DELTA) rb = a.beta[(int64_t)(m0 + min(b0 + tid % DBT, n - 1)) * a.ldb + h];
   };
   fetch(0);
   for (int b0 = 0; b0 < n; b0 += DBT) {
     const int rows = min(DBT, n - b0);
-    lds_barrier();                             // the previous batch's outputs have left
+    lds_barrier();                             // the previous batch's sums have been taken
+    // rows past the sequence: no decay, no key — the state passes them unchanged
 #pragma unroll
     for (int t = 0; t < Q4; ++t) {
       const int e = tid + NT * t, r = e / (DP / 4), i = 4 * (e % (DP / 4));
+      const float pad[3] = {0.f, 0.f, r < rows ? 0.f : 1.f};
 #pragma unroll
-      for (int w = 0; w < 3; ++w) *reinterpret_cast<f32x4*>(&opl[w][r][i]) = rq[w][t];
+      for (int w = OUT ? 0 : 1; w < 3; ++w) {
+        f32x4 x = rq[w][t];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) x[u] = (r < rows && i + u < d) ? x[u] : pad[w];
+        *reinterpret_cast<f32x4*>(&opl[w][r][i]) = x;
+      }
     }
 #pragma unroll
     for (int t = 0; t < NV; ++t) { const int e = tid + NT * t; if (e < DBT * CPB) (&vs[0][0])[e] = rv[t]; }
@@ -409,82 +464,89 @@ __global__ __launch_bounds__(NT) void chan_walk_kernel(ChanArgs a) {
         t = row16_sum(t);
         if ((tid & 15) == 0) bs[1][r] = t;
       }
-      lds_barrier();
     }
-    float qq[NS], kk[NS], gg[NS], v[C], beta = 0.f, kq = 0.f;
-    auto load_row = [&](int r, float (&q_)[NS], float (&k_)[NS], float (&g_)[NS], float (&v_)[C], float& b_, float& kq_) {
+    if (MODE == CHUNK_END && cb == 0) {        // the channels' decay over the chunk
+#pragma unroll
+      for (int t = 0; t < NP; ++t)
+        if (tid + NT * t < DP)
+          for (int r = 0; r < DBT; ++r) gp[t] *= opl[2][r][tid + NT * t];
+    }
+    struct Row { float q[NS], k[NS], g[NS], v[C], beta; } A, B;
+    auto load_row = [&](int r, Row& x) {
 #pragma unroll
       for (int jj = 0; jj < NS / 4; ++jj) {
         const int i = 4 * (s + LPC * jj);
-        const f32x4 q4 = *reinterpret_cast<const f32x4*>(&opl[0][r][i]), k4 = *reinterpret_cast<const f32x4*>(&opl[1][r][i]),
-                    g4 = *reinterpret_cast<const f32x4*>(&opl[2][r][i]);
+        const f32x4 k4 = *reinterpret_cast<const f32x4*>(&opl[1][r][i]), g4 = *reinterpret_cast<const f32x4*>(&opl[2][r][i]);
 #pragma unroll
-        for (int u = 0; u < 4; ++u) { q_[4 * jj + u] = q4[u]; k_[4 * jj + u] = k4[u]; g_[4 * jj + u] = g4[u]; }
+        for (int u = 0; u < 4; ++u) { x.k[4 * jj + u] = k4[u]; x.g[4 * jj + u] = g4[u]; }
+        if (OUT) {
+          const f32x4 q4 = *reinterpret_cast<const f32x4*>(&opl[0][r][i]);
+#pragma unroll
+          for (int u = 0; u < 4; ++u) x.q[4 * jj + u] = q4[u];
+        }
       }
 #pragma unroll
-      for (int cc = 0; cc < C; ++cc) v_[cc] = vs[r][C * cl + cc];
-      if (DELTA) { b_ = bs[0][r]; kq_ = bs[1][r]; }
+      for (int cc = 0; cc < C; ++cc) x.v[cc] = vs[r][C * cl + cc];
+      if (DELTA) x.beta = bs[0][r];
     };
-    load_row(0, qq, kk, gg, v, beta, kq);
-#pragma unroll 2
-    for (int r = 0; r < rows; ++r) {
-      float qn[NS], kn[NS], gn[NS], vn[C], bn = 0.f, kqn = 0.f;
-      load_row(min(r + 1, DBT - 1), qn, kn, gn, vn, bn, kqn);
-      float o[C];
-      if (DELTA) {
-        float pk[C], pq[C];
+    auto step = [&](int r, const Row& x) {
 #pragma unroll
-        for (int cc = 0; cc < C; ++cc) {
-          float k0 = 0.f, k1 = 0.f, q0 = 0.f, q1 = 0.f;
+      for (int cc = 0; cc < C; ++cc) {
+        float q0 = 0.f, q1 = 0.f;
+        if (DELTA) {
 #pragma unroll
-          for (int j = 0; j < NS; j += 2) {
-            S[cc][j] *= gg[j];
-            S[cc][j + 1] *= gg[j + 1];
-            k0 = fmaf(S[cc][j], kk[j], k0); k1 = fmaf(S[cc][j + 1], kk[j + 1], k1);
-            q0 = fmaf(S[cc][j], qq[j], q0); q1 = fmaf(S[cc][j + 1], qq[j + 1], q1);
+          for (int j = 0; j < NS; ++j) S[cc][j] *= x.g[j];
+          float k0 = S[cc][0] * x.k[0], k1 = S[cc][1] * x.k[1];
+#pragma unroll
+          for (int j = 2; j < NS; j += 2) { k0 = fmaf(S[cc][j], x.k[j], k0); k1 = fmaf(S[cc][j + 1], x.k[j + 1], k1); }
+          const float pk = lanes_sum<LPC>(k0 + k1);
+          q0 = S[cc][0] * x.q[0]; q1 = S[cc][1] * x.q[1];
+#pragma unroll
+          for (int j = 2; j < NS; j += 2) { q0 = fmaf(S[cc][j], x.q[j], q0); q1 = fmaf(S[cc][j + 1], x.q[j + 1], q1); }
+          const float u = x.beta * (x.v[cc] - pk);
+#pragma unroll
+          for (int j = 0; j < NS; ++j) S[cc][j] = fmaf(x.k[j], u, S[cc][j]);
+          if (s == 0) us[r][C * cl + cc] = u;
+        } else {
+#pragma unroll
+          for (int j = 0; j < NS; ++j) S[cc][j] = fmaf(x.g[j], S[cc][j], x.k[j] * x.v[cc]);
+          if (OUT) {
+            q0 = S[cc][0] * x.q[0]; q1 = S[cc][1] * x.q[1];
+#pragma unroll
+            for (int j = 2; j < NS; j += 2) { q0 = fmaf(S[cc][j], x.q[j], q0); q1 = fmaf(S[cc][j + 1], x.q[j + 1], q1); }
           }
-          pk[cc] = k0 + k1; pq[cc] = q0 + q1;
         }
-#pragma unroll
-        for (int cc = 0; cc < C; ++cc) { pk[cc] = lanes_sum<LPC>(pk[cc]); pq[cc] = lanes_sum<LPC>(pq[cc]); }
-#pragma unroll
-        for (int cc = 0; cc < C; ++cc) {
-          const float u = beta * (v[cc] - pk[cc]);
-#pragma unroll
-          for (int j = 0; j < NS; ++j) S[cc][j] = fmaf(kk[j], u, S[cc][j]);
-          o[cc] = fmaf(u, kq, pq[cc]);
-        }
-      } else {
-#pragma unroll
-        for (int cc = 0; cc < C; ++cc) {
-          float q0 = 0.f, q1 = 0.f;
-#pragma unroll
-          for (int j = 0; j < NS; j += 2) {
-            S[cc][j] = fmaf(gg[j], S[cc][j], kk[j] * v[cc]);
-            S[cc][j + 1] = fmaf(gg[j + 1], S[cc][j + 1], kk[j + 1] * v[cc]);
-            q0 = fmaf(S[cc][j], qq[j], q0); q1 = fmaf(S[cc][j + 1], qq[j + 1], q1);
-          }
-          o[cc] = q0 + q1;
-        }
-#pragma unroll
-        for (int cc = 0; cc < C; ++cc) o[cc] = lanes_sum<LPC>(o[cc]);
+        if (OUT) part[(r * CPB + C * cl + cc) * PS + s] = q0 + q1;
       }
-      if (s == 0) {
-#pragma unroll
-        for (int cc = 0; cc < C; ++cc) os[r][C * cl + cc] = o[cc] * a.o_scale;
-      }
-#pragma unroll
-      for (int j = 0; j < NS; ++j) { qq[j] = qn[j]; kk[j] = kn[j]; gg[j] = gn[j]; }
-#pragma unroll
-      for (int cc = 0; cc < C; ++cc) v[cc] = vn[cc];
-      beta = bn; kq = kqn;
+    };
+    // two rows per turn, each row's operands requested one step ahead
+    load_row(0, A);
+    for (int r = 0; r < rows; r += 2) {
+      load_row(r + 1, B);
+      step(r, A);
+      load_row(min(r + 2, DBT - 2), A);
+      step(r + 1, B);
     }
+    if (!OUT) continue;
     lds_barrier();
 #pragma unroll
     for (int t = 0; t < NV; ++t) {             // the batch's outputs, a row's columns side by side
       const int e = tid + NT * t, r = e / CPB, cc = cb * CPB + e % CPB;
-      if (r < rows && cc < a.vdim) a.out[(int64_t)(m0 + b0 + r) * a.ldo + (int64_t)h * a.vdim + cc] = (&os[0][0])[e];
+      if (r < rows && cc < a.vdim) {
+        f32x4 o = *reinterpret_cast<const f32x4*>(&part[e * PS]);
+#pragma unroll
+        for (int w = 1; w < LPC / 4; ++w) o += *reinterpret_cast<const f32x4*>(&part[e * PS + 4 * w]);
+        float v = (o[0] + o[1]) + (o[2] + o[3]);
+        if (DELTA) v = fmaf(us[r][e % CPB], bs[1][r], v);
+        a.out[(int64_t)(m0 + b0 + r) * a.ldo + (int64_t)h * a.vdim + cc] = v * a.o_scale;
+      }
     }
+  }
+  if (MODE == CHUNK_OUT) return;
+  if (MODE == CHUNK_END && cb == 0) {
+#pragma unroll
+    for (int t = 0; t < NP; ++t)
+      if (tid + NT * t < d) a.wsp[((int64_t)blockIdx.y * a.H + h) * d + tid + NT * t] = gp[t];
   }
 #pragma unroll
   for (int cc = 0; cc < C; ++cc) {
@@ -495,6 +557,40 @@ __global__ __launch_bounds__(NT) void chan_walk_kernel(ChanArgs a) {
       if (i < d) sp[(int64_t)i * a.vdim + c + cc] = S[cc][j];
     }
   }
+}
+
+// The carry between the chunk passes: grid (ceil(dim vdim / 256), H, n_chunks); the workgroup of a sequence's first chunk in the call turns
+// that sequence's end states into start states, S <- P S + E, and leaves the last state in the arena.
+__global__ __launch_bounds__(256) void chan_carry_kernel(ChanArgs a, int n_chunks) {
+  const int x = blockIdx.x * 256 + threadIdx.x, h = blockIdx.y, c0 = blockIdx.z, de = a.dim * a.vdim, i = x / a.vdim;
+  const int r0 = a.chunk_tab[2 * c0];
+  if (a.row_back[r0] != 0 || x >= de) return;
+  float* sp = a.state + ((int64_t)a.row_seq[r0] * a.H + h) * de + x;
+  float S = a.row_slot[r0] == 0 ? 0.f : *sp;
+  float* w = a.ws + ((int64_t)c0 * a.H + h) * de + x;
+  const float* p = a.wsp + ((int64_t)c0 * a.H + h) * a.dim + i;
+  const int64_t sw = (int64_t)a.H * de, spd = (int64_t)a.H * a.dim;
+  constexpr int PRE = 4;                       // chunks whose states are requested together
+  for (int ch = c0; ch < n_chunks;) {
+    float E[PRE], P[PRE];
+    int cnt = 0;
+#pragma unroll
+    for (int t = 0; t < PRE; ++t) {
+      const int cc = min(ch + t, n_chunks - 1);
+      if (cnt == t && ch + t < n_chunks && (ch + t == c0 || a.row_back[a.chunk_tab[2 * cc]] != 0)) cnt = t + 1;    // the next sequence ends the run
+      E[t] = w[(int64_t)min(t, n_chunks - 1 - ch) * sw];
+      P[t] = p[(int64_t)min(t, n_chunks - 1 - ch) * spd];
+    }
+#pragma unroll
+    for (int t = 0; t < PRE; ++t)
+      if (t < cnt) {
+        w[(int64_t)t * sw] = S;
+        S = fmaf(P[t], S, E[t]);
+      }
+    if (cnt < PRE) break;
+    ch += PRE; w += PRE * sw; p += PRE * spd;
+  }
+  *sp = S;
 }
 
 // The same walk for any head size, the state staying in the arena: grid (ceil(vdim / 32), H, rows or runs), 8 lanes per column.
@@ -592,6 +688,10 @@ __global__ __launch_bounds__(256) void chan_step_kernel(ChanArgs a) {
   if (sub == 0) a.out[(int64_t)m * a.ldo + (int64_t)h * a.vdim + c] = fmaf(u, kq, pq) * a.o_scale;
 }
 
+bool chan_vec(const ChanArgs& a) {
+  return (a.dim & 3) == 0 && (a.ld & 3) == 0 && (a.ldg & 3) == 0 && (((uintptr_t)a.qkv | (uintptr_t)a.g) & 15) == 0;
+}
+
 template <bool DELTA>
 int chan_rows(const ChanArgs& a, bool distinct, int n_runs, hipStream_t st) {
   const int d = a.dim;
@@ -607,9 +707,14 @@ int chan_rows(const ChanArgs& a, bool distinct, int n_runs, hipStream_t st) {
     return MN_OK;
   }
   if (!distinct && d <= 256) {
-#define MN_CW(NS_, LPC_, DB_) \
-  hipLaunchKernelGGL((chan_walk_kernel<NS_, LPC_, 2, 128, DB_, DELTA>), dim3((unsigned)(a.H * mn_cdiv(a.vdim, 128 / LPC_ * 2)), (unsigned)n_runs), dim3(128), 0, st, a)
-    if (d <= 32) MN_CW(4, 8, 16); else if (d <= 64) MN_CW(4, 16, 16); else if (d <= 128) MN_CW(8, 16, 16); else MN_CW(16, 16, 8);
+    const bool vec = chan_vec(a);
+#define MN_CW(NS_, LPC_, NT_, DB_)                                                                                                         \
+  do {                                                                                                                                     \
+    const dim3 grid((unsigned)(a.H * mn_cdiv(a.vdim, NT_ / LPC_)), (unsigned)n_runs);                                                     \
+    if (vec) hipLaunchKernelGGL((chan_walk_kernel<NS_, LPC_, 1, NT_, DB_, DELTA, true, WALK>), grid, dim3(NT_), 0, st, a);                \
+    else hipLaunchKernelGGL((chan_walk_kernel<NS_, LPC_, 1, NT_, DB_, DELTA, false, WALK>), grid, dim3(NT_), 0, st, a);                   \
+  } while (0)
+    if (d <= 32) MN_CW(4, 8, 128, 16); else if (d <= 64) MN_CW(4, 16, 128, 16); else if (d <= 128) MN_CW(8, 16, 128, 16); else MN_CW(16, 16, 128, 8);
 #undef MN_CW
     MN_CHECK_LAUNCH("mn_channel_state_rows(walk)");
     return MN_OK;
@@ -694,6 +799,9 @@ extern "C" int mn_token_table_rows(const int32_t* table, int vocab, int top, con
   return MN_OK;
 }
 
+extern "C" size_t mn_sizeof_low_rank_job(void) { return sizeof(mn_low_rank_job); }
+extern "C" size_t mn_sizeof_rows_prep(void) { return sizeof(mn_rows_prep); }
+
 namespace {
 bool low_rank_ok(const mn_low_rank_job& j) {
   return j.a && j.w && j.out && j.k >= 1 && j.n >= 1 && j.kind >= MN_LOW_RANK_LINEAR && j.kind <= MN_LOW_RANK_SIGMOID &&
@@ -708,7 +816,7 @@ extern "C" int mn_low_rank_gate_rows(const mn_low_rank_job* jobs, int n_jobs, in
   a.job[0] = jobs[0];
   a.job[1] = jobs[n_jobs - 1];
   a.M = M;
-  const bool few = M <= 2 * LR_ROWS;
+  const bool few = M <= 64;
   const int tile = few ? 32 : 64, rows = few ? LR_ROWS : 64;
   a.nb0 = (int)mn_cdiv(jobs[0].n, tile);
   const dim3 grid((unsigned)(a.nb0 + (n_jobs == 2 ? mn_cdiv(jobs[1].n, tile) : 0)), (unsigned)mn_cdiv(M, rows));
@@ -716,6 +824,40 @@ extern "C" int mn_low_rank_gate_rows(const mn_low_rank_job* jobs, int n_jobs, in
   if (few) hipLaunchKernelGGL(low_rank_few_kernel, grid, dim3(256), 0, mn_stream(stream), a);
   else hipLaunchKernelGGL(low_rank_mfma_kernel, grid, dim3(256), 0, mn_stream(stream), a);
   MN_CHECK_LAUNCH("mn_low_rank_gate_rows");
+  return MN_OK;
+}
+
+extern "C" int mn_rows_prep_launch(const mn_rows_prep* p, const int32_t* row_seq, const int32_t* row_slot, int M, void* stream) {
+  MN_CHECK_ARG(p && M >= 1 && M <= 64 && p->n_jobs >= 0 && p->n_jobs <= 2 && p->act_n >= 0 && p->top >= 0, "mn_rows_prep_launch: bad args (M=%d: at most 64)", M);
+  MN_CHECK_ARG(!p->delta || (p->proj && p->w_conv && row_seq && row_slot && p->qkv && p->beta && p->H >= 1 && p->G >= 1 && (p->H % p->G) == 0 &&
+                             p->dim >= 1 && p->vdim >= 1 && p->taps >= 1 && (p->taps == 1 || p->conv_state) && p->ldbeta >= p->H),
+               "mn_rows_prep_launch: bad delta-rule args");
+  for (int i = 0; i < p->n_jobs; ++i) MN_CHECK_ARG(low_rank_ok(p->job[i]), "mn_rows_prep_launch: job %d: bad sizes or null operands", i);
+  MN_CHECK_ARG(p->act_n == 0 || (p->act_x && p->act_y), "mn_rows_prep_launch: the activation needs its rows");
+  MN_CHECK_ARG(p->top == 0 || (p->table && p->tok && p->idx && p->vocab >= 1), "mn_rows_prep_launch: the table needs its rows");
+  RowsPrepArgs a{};
+  a.M = M;
+  if (p->delta) {
+    a.delta = DeltaPrepArgs{p->proj, p->ld, p->H, p->G, p->dim, p->vdim, p->taps, p->off_b, 0, p->w_conv, p->conv_state, 1, nullptr, nullptr, p->unit_eps,
+                            p->q_scale, row_seq, row_slot, nullptr, p->qkv, p->ldqkv, p->beta, p->ldbeta};
+    a.n_delta = (int)mn_cdiv(delta_prep_units(p->H, p->G, p->vdim), 4);
+  }
+  if (p->n_jobs > 0) {
+    a.lr.job[0] = p->job[0];
+    a.lr.job[1] = p->job[p->n_jobs - 1];
+    a.lr.M = M;
+    a.lr.nb0 = (int)mn_cdiv(p->job[0].n, 32);
+    a.n_lr = a.lr.nb0 + (p->n_jobs == 2 ? (int)mn_cdiv(p->job[1].n, 32) : 0);
+  }
+  if (p->act_n > 0) {
+    a.act = XieluArgs{p->act_x, p->ld_act_x, p->act_pos, p->act_neg, p->act_y, p->ld_act_y, nullptr, 0, M, p->act_n};
+    a.n_act = (int)mn_cdiv(p->act_n, 1024);
+  }
+  a.table = p->table; a.tok = p->tok; a.vocab = p->vocab; a.top = p->top; a.idx = p->idx;
+  const int64_t blocks = (int64_t)a.n_delta + a.n_lr + a.n_act + (p->top > 0 ? 1 : 0);
+  if (blocks == 0) return MN_OK;
+  hipLaunchKernelGGL(rows_prep_kernel, dim3((unsigned)blocks, (unsigned)M), dim3(256), 0, mn_stream(stream), a);
+  MN_CHECK_LAUNCH("mn_rows_prep_launch");
   return MN_OK;
 }
 
@@ -728,9 +870,45 @@ extern "C" int mn_channel_state_rows(const float* qkv, int64_t ld, const float* 
                "mn_channel_state_rows: bad args (dim=%d: at most 4096)", dim);
   MN_CHECK_ARG(!blk_tab || (n_blk >= 1 && n_blk <= M), "mn_channel_state_rows: bad table of runs");
   ChanArgs a{qkv, ld, g, ldg, beta, ldb, H, G, dim, vdim, o_scale, state, row_seq, row_slot, distinct ? nullptr : row_back, distinct ? nullptr : blk_tab,
-             out, ldo, M};
+             out, ldo, M, nullptr, nullptr, nullptr};
   const int n_runs = a.blk_tab ? n_blk : M;
   return beta ? chan_rows<true>(a, distinct, n_runs, mn_stream(stream)) : chan_rows<false>(a, distinct, n_runs, mn_stream(stream));
+}
+
+extern "C" int mn_channel_chunk_rows(void) { return 128; }
+
+extern "C" size_t mn_channel_scan_workspace_bytes(int n_chunks, int H, int dim, int vdim) {
+  if (n_chunks < 1 || H < 1 || dim < 1 || vdim < 1) return 0;
+  return (size_t)n_chunks * H * dim * ((size_t)vdim + 1) * sizeof(float);
+}
+
+extern "C" int mn_channel_state_rows_scan(const float* qkv, int64_t ld, const float* g, int64_t ldg, int M, int H, int G, int dim, int vdim,
+                                          float o_scale, float* state, const int32_t* row_seq, const int32_t* row_slot, const int32_t* row_back,
+                                          const int32_t* chunk_tab, int n_chunks, float* out, int64_t ldo, void* workspace,
+                                          size_t workspace_bytes, void* stream) {
+  MN_CHECK_ARG(qkv && g && state && row_seq && row_slot && row_back && chunk_tab && out && workspace && M >= 1 && H >= 1 && H <= 65535 && G >= 1 &&
+                   (H % G) == 0 && dim >= 1 && dim <= 256 && vdim >= 1 && n_chunks >= 1 && n_chunks <= 65535,
+               "mn_channel_state_rows_scan: bad args (dim=%d: at most 256)", dim);
+  MN_CHECK_ARG(workspace_bytes >= mn_channel_scan_workspace_bytes(n_chunks, H, dim, vdim), "mn_channel_state_rows_scan: workspace too small");
+  float* ws = (float*)workspace;
+  ChanArgs a{qkv, ld, g, ldg, nullptr, 0, H, G, dim, vdim, o_scale, state, row_seq, row_slot, row_back, nullptr, out, ldo, M, chunk_tab, ws,
+             ws + (size_t)n_chunks * H * dim * vdim};
+  hipStream_t st = mn_stream(stream);
+  const bool vec = chan_vec(a);
+  const dim3 carry((unsigned)mn_cdiv((int64_t)dim * vdim, 256), (unsigned)H, (unsigned)n_chunks);
+#define MN_CS(NS_, LPC_, DB_)                                                                                                              \
+  do {                                                                                                                                     \
+    const dim3 grid((unsigned)(H * mn_cdiv(vdim, 128 / LPC_ * 2)), (unsigned)n_chunks);                                                   \
+    if (vec) hipLaunchKernelGGL((chan_walk_kernel<NS_, LPC_, 2, 128, DB_, false, true, CHUNK_END>), grid, dim3(128), 0, st, a);           \
+    else hipLaunchKernelGGL((chan_walk_kernel<NS_, LPC_, 2, 128, DB_, false, false, CHUNK_END>), grid, dim3(128), 0, st, a);              \
+    hipLaunchKernelGGL(chan_carry_kernel, carry, dim3(256), 0, st, a, n_chunks);                                                          \
+    if (vec) hipLaunchKernelGGL((chan_walk_kernel<NS_, LPC_, 2, 128, DB_, false, true, CHUNK_OUT>), grid, dim3(128), 0, st, a);           \
+    else hipLaunchKernelGGL((chan_walk_kernel<NS_, LPC_, 2, 128, DB_, false, false, CHUNK_OUT>), grid, dim3(128), 0, st, a);              \
+  } while (0)
+  if (dim <= 32) MN_CS(4, 8, 16); else if (dim <= 64) MN_CS(4, 16, 16); else if (dim <= 128) MN_CS(8, 16, 16); else MN_CS(16, 16, 8);
+#undef MN_CS
+  MN_CHECK_LAUNCH("mn_channel_state_rows_scan");
+  return MN_OK;
 }
 
 extern "C" int mn_gemv_glu_indexed(const float* A, int64_t lda, int a_div, const uint16_t* W, int64_t ldw, int64_t w_bs, const int32_t* w_idx,

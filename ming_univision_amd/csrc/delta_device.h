@@ -48,10 +48,10 @@ __device__ __forceinline__ float conv_silu(const DeltaPrepArgs& a, int m, int c,
   return silu_x(acc);
 }
 
-// one wave: unit < 2 G = a q or k head of row m (its unit norm is a wave's reduction), then 256 value channels per unit
-__device__ __forceinline__ void delta_prep_unit(const DeltaPrepArgs& a, int m, int unit, int lane) {
+// one wave (back: rows of the same sequence directly before row m in this call): unit < 2 G = a q or k head of row m (its unit norm is a wave's reduction), then 256 value channels per unit
+__device__ __forceinline__ void delta_prep_unit(const DeltaPrepArgs& a, int m, int unit, int lane, int back) {
   const int nqk = 2 * a.G * a.dim, nv = a.H * a.vdim, n = nqk + nv;
-  const int seq = a.row_seq[m], slot = a.row_slot[m], back = a.row_back[m];
+  const int seq = a.row_seq[m], slot = a.row_slot[m];
   float* out = a.qkv + (int64_t)m * a.ldo;
   if (unit < 2 * a.G) {
     const int c0 = unit * a.dim;

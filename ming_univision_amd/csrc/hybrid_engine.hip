@@ -5,8 +5,8 @@
 //   mixer    attention:      head norms + temperature + append, then the block attention with the heads' sinks
 //            lightning:      the recurrence (row by row, one decode row cut over many workgroups, or the chunked scan), RMS x sigmoid gate
 //            talk attention: rotation + unit norms + append (values = the projected keys), the attention with mixed heads
-//            channel delta:  filters + silu + unit norms + write strengths; the low-rank decays and gates in one launch; the recurrence;
-//                            per-head RMS x gate
+//            channel delta:  filters + silu + unit norms + write strengths; the low-rank decays and gates in one launch (decode rows: all
+//                            of this and the feed-forward's activation in one launch); the recurrence; per-head RMS x gate
 //            gla:            the low-rank decays, the recurrence straight from the stacked product, per-head RMS x silu gate
 //   x += [mixer | act(up)] [W_o | W_down]^T        ONE product for the mixer's output and the dense / shared expert's down projection
 //   experts of a mixture: as in pmix_engine.hip (sorted by expert on the grouped MFMA GEMMs, or pair by pair on fp32 FMA); picks that
@@ -60,7 +60,8 @@ HDims hdims(const mn_hyb_layer& l) {
 struct HPlan {
   int n_in = 1, cq = 1, hv = 1, n_cat = 1, top = 1, eff = 1, eup = 1, experts = 1, dec = 1, gate = 1, beta = 1;
   size_t gemm_ws = 0, attn_ws = 0;
-  int64_t lin = 0;                                               // largest heads x dim x vdim of a recurrence
+  int64_t lin = 0;                                               // largest heads x dim x vdim of a lightning recurrence
+  size_t gla = 0;                                                // largest bytes of a gla layer's chunk state
 };
 
 enum { EXPERTS_INDEXED = 0, EXPERTS_GROUPED = 1, EXPERTS_TILES = 2 };
@@ -103,6 +104,9 @@ HPlan make_plan(const mn_hyb_model* m, int M) {
     } else if (l.kind == MN_HYB_LIGHTNING) {
       const int64_t s = (int64_t)l.heads * l.dim * l.vdim;
       if (s > p.lin) p.lin = s;
+    } else if (l.kind == MN_HYB_GLA) {
+      const size_t s = mn_channel_scan_workspace_bytes(1, l.heads, l.dim, l.vdim);
+      if (s > p.gla) p.gla = s;
     }
     if (m->arith == MN_SEQ_ARITH_BF16 && M > 8 && M <= 64) {       // scratch of the weight-streaming MFMA route: the largest product of the stack
       const int W = m->width;
@@ -117,11 +121,13 @@ HPlan make_plan(const mn_hyb_model* m, int M) {
   return p;
 }
 
-// chunk states the scan of a step may hold: full chunks plus one ragged chunk for each of up to 64 sequences; steps too short for the
+// chunk states the scans of a step may hold: full chunks plus one ragged chunk for each of up to 64 sequences; steps too short for a
 // scan hold none
 inline size_t scan_bytes(const HPlan& p, int M) {
-  const int c = mn_lightning_chunk_rows();
-  return M >= 2 * c ? (size_t)(mn_cdiv(M, c) + 64) * (size_t)p.lin * sizeof(float) : 0;
+  const int c = mn_lightning_chunk_rows(), g = mn_channel_chunk_rows();
+  const size_t light = M >= 2 * c ? (size_t)(mn_cdiv(M, c) + 64) * (size_t)p.lin * sizeof(float) : 0;
+  const size_t chan = M >= 2 * g ? (size_t)(mn_cdiv(M, g) + 64) * p.gla : 0;
+  return light > chan ? light : chan;
 }
 
 }  // namespace
@@ -253,6 +259,29 @@ extern "C" int mn_hyb_step(const mn_hyb_model* m, const mn_hyb_state* st, const 
     const bool cat16_only = cath && mfma_ok(l.w_out, d.n_cat);
     MN_TRY(norm_stage(l.norm1, h16_only ? nullptr : hf, hh));
     MN_TRY(linear(arith, M, hf, W, hh, W, l.w_in, d.n_in, W, nullptr, pin, d.n_in, gws, gwb, stream));
+    // ---- decode rows of the channel-decay mixers: what depends on the stacked product alone, in one launch ----
+    const int E = l.experts, top = l.top, eff = l.expert_ff, Z = M * top;
+    const bool prepped = one_row && M <= 64 && !cath && (delta || gla) && (d.n_up == 0 || l.ff_act == MN_HYB_ACT_XIELU) && (!moe || (l.table && layer_norm));
+    const mn_low_rank_job jobs[2] = {
+        {pin + d.off_a1, d.n_in, l.w_a2, l.b_a2, l.a_log, dec, d.n_dec, l.rank_a, d.n_dec, delta ? MN_LOW_RANK_DECAY : MN_LOW_RANK_ROOT, l.dim, l.root},
+        {pin + d.off_g1, d.n_in, l.w_g2, nullptr, nullptr, gat, d.hv, l.rank_g, d.hv, MN_LOW_RANK_SIGMOID, 1, 1.0f}};
+    const float unit_scale = 1.0f / sqrtf((float)l.dim);
+    if (prepped) {
+      mn_rows_prep r;
+      memset(&r, 0, sizeof(r));
+      if (delta) {
+        r.delta = 1; r.proj = pin; r.ld = d.n_in; r.H = l.heads; r.G = l.kv_heads; r.dim = l.dim; r.vdim = l.vdim; r.taps = l.conv; r.off_b = d.off_b;
+        r.w_conv = l.w_conv; r.conv_state = st->conv[ri]; r.unit_eps = l.unit_eps; r.q_scale = unit_scale;
+        r.qkv = qf; r.ldqkv = d.cq; r.beta = bet; r.ldbeta = l.heads;
+      }
+      r.n_jobs = delta ? 2 : 1; r.job[0] = jobs[0]; r.job[1] = jobs[1];
+      if (d.n_up > 0) {
+        r.act_x = pin + d.off_up; r.ld_act_x = d.n_in; r.act_pos = l.act_pos; r.act_neg = l.act_neg;
+        r.act_y = cat + d.hv; r.ld_act_y = d.n_cat; r.act_n = d.n_up;
+      }
+      if (moe) { r.table = l.table; r.tok = row_tok; r.vocab = m->vocab; r.top = top; r.idx = tidx; }
+      MN_TRY(mn_rows_prep_launch(&r, row_seq, row_slot, M, stream));
+    }
     // ---- mixer ----
     if (attn) {
       MN_TRY(mn_head_norm_temp_append(pin, d.n_in, M, l.heads, l.kv_heads, l.dim, l.vdim, l.q_norm, l.k_norm, m->eps, l.scale, l.temp_coef,
@@ -275,23 +304,25 @@ extern "C" int mn_hyb_step(const mn_hyb_model* m, const mn_hyb_state* st, const 
                           l.heads, l.kv_heads, l.dim, st->t_max, l.window, l.chunk, cat16_only ? nullptr : cat, d.n_cat, cath, d.n_cat, ns, aws,
                           p.attn_ws, -1, stream));
     } else if (delta) {
-      MN_TRY(mn_delta_prep_rows(pin, d.n_in, M, l.heads, l.kv_heads, l.dim, l.vdim, d.off_b, 0, l.w_conv, l.conv, st->conv[ri], one_row ? 1 : 0,
-                                nullptr, nullptr, l.unit_eps, 1.0f / sqrtf((float)l.dim), row_seq, row_slot, row_back, qf, d.cq, bet, l.heads,
-                                stream));
-      if (l.conv > 1 && !one_row) MN_TRY(mn_tap_state_update(pin, d.n_in, l.conv, st->conv[ri], row_seq, row_back, M, d.cq, stream));
-      const mn_low_rank_job jobs[2] = {
-          {pin + d.off_a1, d.n_in, l.w_a2, l.b_a2, l.a_log, dec, d.n_dec, l.rank_a, d.n_dec, MN_LOW_RANK_DECAY, l.dim, 1.0f},
-          {pin + d.off_g1, d.n_in, l.w_g2, nullptr, nullptr, gat, d.hv, l.rank_g, d.hv, MN_LOW_RANK_SIGMOID, 1, 1.0f}};
-      MN_TRY(mn_low_rank_gate_rows(jobs, 2, M, stream));
+      if (!prepped) {
+        MN_TRY(mn_delta_prep_rows(pin, d.n_in, M, l.heads, l.kv_heads, l.dim, l.vdim, d.off_b, 0, l.w_conv, l.conv, st->conv[ri], one_row ? 1 : 0,
+                                  nullptr, nullptr, l.unit_eps, unit_scale, row_seq, row_slot, row_back, qf, d.cq, bet, l.heads, stream));
+        if (l.conv > 1 && !one_row) MN_TRY(mn_tap_state_update(pin, d.n_in, l.conv, st->conv[ri], row_seq, row_back, M, d.cq, stream));
+        MN_TRY(mn_low_rank_gate_rows(jobs, 2, M, stream));
+      }
       MN_TRY(mn_channel_state_rows(qf, d.cq, dec, d.n_dec, bet, l.heads, M, l.heads, l.kv_heads, l.dim, l.vdim, 1.0f, st->lin[ri], row_seq, row_slot,
                                    row_back, blk_tab, n_blk, one_row ? MN_SEQ_ROWS_DISTINCT : 0, lo, d.hv, stream));
       MN_TRY(mn_head_rms_gate_rows(lo, d.hv, l.mix_norm, m->eps, gat, d.hv, MN_GATE_ACT_NONE, cat16_only ? nullptr : cat, d.n_cat, cath, d.n_cat, M,
                                    l.heads, l.vdim, stream));
     } else if (gla) {
-      const mn_low_rank_job job = {pin + d.off_a1, d.n_in, l.w_a2, l.b_a2, nullptr, dec, d.n_dec, l.rank_a, d.n_dec, MN_LOW_RANK_ROOT, 1, l.root};
-      MN_TRY(mn_low_rank_gate_rows(&job, 1, M, stream));
-      MN_TRY(mn_channel_state_rows(pin, d.n_in, dec, d.n_dec, nullptr, 0, M, l.heads, l.heads, l.dim, l.vdim, 1.0f / sqrtf((float)l.dim), st->lin[ri],
-                                   row_seq, row_slot, row_back, blk_tab, n_blk, one_row ? MN_SEQ_ROWS_DISTINCT : 0, lo, d.hv, stream));
+      if (!prepped) MN_TRY(mn_low_rank_gate_rows(jobs, 1, M, stream));
+      if (!one_row && chunk_tab && n_chunks >= 1 && M >= 2 * mn_channel_chunk_rows() && l.dim <= 256 &&
+          mn_channel_scan_workspace_bytes(n_chunks, l.heads, l.dim, l.vdim) <= scan_cap)
+        MN_TRY(mn_channel_state_rows_scan(pin, d.n_in, dec, d.n_dec, M, l.heads, l.heads, l.dim, l.vdim, unit_scale, st->lin[ri], row_seq, row_slot,
+                                          row_back, chunk_tab, n_chunks, lo, d.hv, scanws, scan_cap, stream));
+      else
+        MN_TRY(mn_channel_state_rows(pin, d.n_in, dec, d.n_dec, nullptr, 0, M, l.heads, l.heads, l.dim, l.vdim, unit_scale, st->lin[ri], row_seq,
+                                     row_slot, row_back, blk_tab, n_blk, one_row ? MN_SEQ_ROWS_DISTINCT : 0, lo, d.hv, stream));
       MN_TRY(mn_head_rms_gate_rows(lo, d.hv, l.mix_norm, m->eps, pin + d.off_g, d.n_in, MN_GATE_ACT_SILU, cat16_only ? nullptr : cat, d.n_cat, cath,
                                    d.n_cat, M, l.heads, l.vdim, stream));
     } else {
@@ -307,13 +338,12 @@ extern "C" int mn_hyb_step(const mn_hyb_model* m, const mn_hyb_state* st, const 
       MN_TRY(mn_rms_sigmoid_gate_rows(lo, d.hv, l.mix_norm, m->eps, pin + d.off_g, d.n_in, cat, d.n_cat, cath, d.n_cat, M, d.hv, stream));
     }
     // ---- the feed-forward's activation and router; the joined output product ----
-    const int E = l.experts, top = l.top, eff = l.expert_ff, Z = M * top;
-    if (moe && l.table) MN_TRY(mn_token_table_rows(l.table, m->vocab, top, row_tok, M, tidx, layer_norm ? nullptr : tw, stream));
+    if (moe && l.table && !prepped) MN_TRY(mn_token_table_rows(l.table, m->vocab, top, row_tok, M, tidx, layer_norm ? nullptr : tw, stream));
     const bool ride = moe && !l.table && d.n_up > 0 && !cath && l.ff_act == MN_HYB_ACT_RELU2;   // few rows: the shared activation rides the router's launch
     if (moe && !l.table)
       MN_TRY(mn_router_softmax_topk_rows(pin + d.off_router, d.n_in, M, d.n_router, E, top, l.correction, tidx, tw, ride ? pin + d.off_up : nullptr,
                                          d.n_in, ride ? cat + d.hv : nullptr, d.n_cat, ride ? d.n_up : 0, stream));
-    if (d.n_up > 0 && !ride) {
+    if (d.n_up > 0 && !ride && !prepped) {
       float* ay = cat16_only ? nullptr : cat + d.hv;
       uint16_t* ah = cath ? cath + d.hv : nullptr;
       if (l.ff_act == MN_HYB_ACT_XIELU)

@@ -203,7 +203,7 @@ __global__ __launch_bounds__(256) void head_sigmoid_gate_kernel(float* __restric
 // ---------------------------------------------------------------------------------------------------------------------------
 // grid (M, ceil(units / 4)): a wave takes one unit of a row — a q or k head (its unit norm is a wave's reduction) or 256 value channels
 __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrepArgs a) {
-  delta_prep_unit(a, blockIdx.x, blockIdx.y * 4 + (threadIdx.x >> 6), threadIdx.x & 63);
+  delta_prep_unit(a, blockIdx.x, blockIdx.y * 4 + (threadIdx.x >> 6), threadIdx.x & 63, a.row_back[blockIdx.x]);
   if (blockIdx.y == 0) delta_prep_strengths(a, blockIdx.x, threadIdx.x);
 }
 
@@ -366,6 +366,7 @@ __global__ __launch_bounds__(256) void delta_rows_fast_kernel(DeltaArgs a) {
     const int i = 4 * (s + LPC * (j >> 2)) + (j & 3);
     S[j] = (on && !fresh && i < d) ? sp[(int64_t)i * a.vdim] : 0.f;
   }
+  __syncthreads();                           // the state has arrived: from here on only a batch's loads are in flight
   float* qk = lds;                           // row r: q at r * 2 DP, k at r * 2 DP + DP
   float* vs = qk + DBT * 2 * DP;
   float* bs = vs + DBT * CPB;

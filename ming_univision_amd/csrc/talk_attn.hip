@@ -14,7 +14,7 @@ struct TalkArgs {
   const float *k, *v; int64_t ldk, ldv;        // arenas [n_seq, t_max, ld]
   const float *talk, *sink;                    // [H, H]; [H] or NULL
   const int32_t *row_seq, *row_slot, *blk_tab;
-  int H, G, dim, t_max, window, chunk, rows, nsplit, vec;
+  int H, G, dim, t_max, window, chunk, rows, nsplit, ovec;
   float* out; int64_t ldo; bf16_t* out16; int64_t ldo16;
   float* part;
 };
@@ -33,19 +33,9 @@ __device__ __forceinline__ float talk_inv(float m, float l, const float* sink, i
   return f / (l * f + expf(sk - mm));
 }
 
-__device__ __forceinline__ f32x4 ld4(const float* row, int d, int dim, int vec) {
-  if (vec) {
-    const f32x4 t = *reinterpret_cast<const f32x4*>(row + (d < dim ? d : 0));
-    return d < dim ? t : f32x4{0.f, 0.f, 0.f, 0.f};
-  }
-  f32x4 r;
-#pragma unroll
-  for (int u = 0; u < 4; ++u) {
-    const float t = row[d + u < dim ? d + u : 0];
-    r[u] = d + u < dim ? t : 0.f;
-  }
-  return r;
-}
+// 16 bytes of a row of `dim` (a multiple of 4) values; past its end the row's last ones.  Keys need no mask there (the queries are zero
+// padded) and neither do values (their columns are not written), so every load stands alone in the instruction stream.
+__device__ __forceinline__ f32x4 ld4(const float* row, int d, int dim) { return *reinterpret_cast<const f32x4*>(row + min(d, dim - 4)); }
 
 // Matrix-core form (v_mfma_f32_16x16x4_f32: scores, mixing and values stay fp32).  A workgroup of 4 waves owns a run of up to `rows` rows
 // of one sequence with all heads; the query vectors (row, head) of a key/value head form TV tiles of 16 (vector r rep + head % rep).  A
@@ -96,8 +86,8 @@ __global__ __launch_bounds__(256, (KW * TW * NBD <= 2 && HB == 1 ? 2 : 1)) void 
       const float* src = a.q + (int64_t)(r0 + (on ? r : 0)) * a.ldq + (int64_t)(on ? kap[x] * rep + vv % rep : 0) * a.dim;
 #pragma unroll
       for (int j = 0; j < ND; ++j) {
-        const f32x4 t = ld4(src, 16 * j + 4 * g4, a.dim, a.vec);
-        qreg[x * TW + w][j] = on ? t : f32x4{0.f, 0.f, 0.f, 0.f};
+        const f32x4 t = ld4(src, 16 * j + 4 * g4, a.dim);
+        qreg[x * TW + w][j] = (on && 16 * j + 4 * g4 < a.dim) ? t : f32x4{0.f, 0.f, 0.f, 0.f};
         acc[x * TW + w][j] = f32x4{0.f, 0.f, 0.f, 0.f};
       }
     }
@@ -109,7 +99,7 @@ __global__ __launch_bounds__(256, (KW * TW * NBD <= 2 && HB == 1 ? 2 : 1)) void 
     for (int x = 0; x < KW; ++x)
       if (kap[x] >= 0) {
 #pragma unroll
-        for (int j = 0; j < ND; ++j) kreg[x][j] = ld4(row + (int64_t)kap[x] * a.dim, 16 * j + 4 * g4, a.dim, a.vec);
+        for (int j = 0; j < ND; ++j) kreg[x][j] = ld4(row + (int64_t)kap[x] * a.dim, 16 * j + 4 * g4, a.dim);
       }
   };
   auto fetch_v = [&](int tile) {
@@ -120,7 +110,7 @@ __global__ __launch_bounds__(256, (KW * TW * NBD <= 2 && HB == 1 ? 2 : 1)) void 
         for (int t = 0; t < 4; ++t) {
           const float* row = vb + (int64_t)min(16 * tile + t + 4 * g4, nk - 1) * a.ldv + (int64_t)kap[x] * a.dim;
 #pragma unroll
-          for (int j = 0; j < NBD; ++j) vreg[x][t][j] = ld4(row, 64 * j + 4 * c16, a.dim, a.vec);
+          for (int j = 0; j < NBD; ++j) vreg[x][t][j] = ld4(row, 64 * j + 4 * c16, a.dim);
         }
       }
   };
@@ -245,19 +235,29 @@ __global__ __launch_bounds__(256, (KW * TW * NBD <= 2 && HB == 1 ? 2 : 1)) void 
         const float inv = part ? 1.0f : Cl[vid];
         const int64_t col0 = (int64_t)(kap[x] * rep + vv % rep) * a.dim;
 #pragma unroll
-        for (int j = 0; j < NBD; ++j)
+        for (int j = 0; j < NBD; ++j) {
+          const int d = 64 * j + 4 * c16;
+          if (d >= a.dim) continue;
+          f32x4 val;
 #pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            const int d = 64 * j + 4 * c16 + e;
-            if (d >= a.dim) continue;
-            const float val = acc[x * TW + w][4 * j + e][i] * inv;
-            if (part) {
-              part[2 * NV + (int64_t)vid * a.dim + d] = val;
-            } else {
-              if (a.out) a.out[(int64_t)(r0 + r) * a.ldo + col0 + d] = val;
-              if (a.out16) a.out16[(int64_t)(r0 + r) * a.ldo16 + col0 + d] = f32_to_bf16(val);
+          for (int e = 0; e < 4; ++e) val[e] = acc[x * TW + w][4 * j + e][i] * inv;
+          if (part) {
+            *reinterpret_cast<f32x4*>(part + 2 * NV + (int64_t)vid * a.dim + d) = val;
+            continue;
+          }
+          const int64_t row = r0 + r;
+          if (a.ovec) {
+            if (a.out) *reinterpret_cast<f32x4*>(a.out + row * a.ldo + col0 + d) = val;
+            if (a.out16)
+              *reinterpret_cast<uint2*>(a.out16 + row * a.ldo16 + col0 + d) = make_uint2(pack_bf16x2(val[0], val[1]), pack_bf16x2(val[2], val[3]));
+          } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              if (a.out) a.out[row * a.ldo + col0 + d + e] = val[e];
+              if (a.out16) a.out16[row * a.ldo16 + col0 + d + e] = f32_to_bf16(val[e]);
             }
           }
+        }
       }
     }
   }
@@ -290,8 +290,8 @@ __global__ __launch_bounds__(256) void talk_attn_merge_kernel(TalkArgs a) {
     const int i = e / cw, d = c0 + e - i * cw, vv = 16 * vt + i;
     const float* src = base + 2 * NV + (int64_t)(kap * TV * 16 + vv) * a.dim + d;
     float t = 0.f;
-#pragma unroll 4
-    for (int s = 0; s < a.nsplit; ++s) t = wgt[i][s] != 0.f ? fmaf(src[s * stride], wgt[i][s], t) : t;
+#pragma unroll 8
+    for (int s = 0; s < a.nsplit; ++s) t = fmaf(src[s * stride], wgt[i][s], t);      // a split without keys left zeros
     const float val = t * inv[i];
     const int64_t col = (int64_t)(kap * rep + vv % rep) * a.dim + d;
     if (a.out) a.out[(int64_t)(r0 + vv / rep) * a.ldo + col] = val;
@@ -364,7 +364,7 @@ __global__ __launch_bounds__(PLAIN_NT) void talk_attn_plain_kernel(TalkArgs a) {
 struct TalkShape { int nbd, kw, tw, hb; };      // nbd 0: no matrix-core instance
 TalkShape talk_shape(int H, int G, int dim, int rows) {
   TalkShape s{0, 0, 0, 0};
-  if (H < 1 || G < 1 || (H % G) != 0 || dim < 1 || rows < 1) return s;
+  if (H < 1 || G < 1 || (H % G) != 0 || dim < 4 || (dim % 4) != 0 || rows < 1) return s;
   const int rep = H / G, TV = (rows * rep + 15) / 16;
   const int nbd = dim <= 64 ? 1 : (dim <= 128 ? 2 : (dim <= 256 ? 4 : 0)), hb = H <= 16 ? 1 : (H <= 32 ? 2 : (H <= 64 ? 4 : 0));
   if (!nbd || !hb || rows > 8 || (hb == 4 && rows > 4)) return s;
@@ -413,15 +413,15 @@ extern "C" int mn_talk_attn(const float* q, int64_t ldq, const float* k_arena, i
   MN_CHECK_ARG(variant >= -1 && variant <= MN_TALK_ATTN_PLAIN, "mn_talk_attn: unknown variant %d", variant);
   const TalkShape s = talk_shape(H, G, dim, rows);
   const size_t lds = s.nbd ? talk_lds(H, G, rows, s.hb) : 0;
-  const bool fits = s.nbd && lds <= 64 * 1024;
+  const bool fits = s.nbd && lds <= 64 * 1024 && (ldq % 4) == 0 && (ldk % 4) == 0 && (ldv % 4) == 0 &&
+                    (((uintptr_t)q | (uintptr_t)k_arena | (uintptr_t)v_arena | (uintptr_t)workspace) & 15) == 0;
   if (variant < 0) variant = fits ? MN_TALK_ATTN_MFMA : MN_TALK_ATTN_PLAIN;
   MN_CHECK_ARG(variant == MN_TALK_ATTN_PLAIN || fits, "mn_talk_attn: no matrix-core instance for H=%d G=%d dim=%d rows=%d", H, G, dim, rows);
   if (variant == MN_TALK_ATTN_PLAIN) nsplit = 1;
   MN_CHECK_ARG(nsplit >= 1 && nsplit <= 64 && (nsplit == 1 || (workspace && workspace_bytes >= mn_talk_attn_workspace_bytes(n_blk, H, G, dim, rows, nsplit))),
                "mn_talk_attn: 1 .. 64 key splits with their workspace");
-  const int vec = (dim % 4) == 0 && (ldq % 4) == 0 && (ldk % 4) == 0 && (ldv % 4) == 0 &&
-                  (((uintptr_t)q | (uintptr_t)k_arena | (uintptr_t)v_arena) & 15) == 0;
-  TalkArgs a{q, ldq, k_arena, v_arena, ldk, ldv, talk, sink, row_seq, row_slot, blk_tab, H, G, dim, t_max, window, chunk, rows, nsplit, vec,
+  const int ovec = (!out || ((ldo % 4) == 0 && (((uintptr_t)out) & 15) == 0)) && (!out16 || ((ldo16 % 4) == 0 && (((uintptr_t)out16) & 7) == 0));
+  TalkArgs a{q, ldq, k_arena, v_arena, ldk, ldv, talk, sink, row_seq, row_slot, blk_tab, H, G, dim, t_max, window, chunk, rows, nsplit, ovec,
              out, ldo, out16, ldo16, (float*)workspace};
   hipStream_t st = mn_stream(stream);
   if (variant == MN_TALK_ATTN_PLAIN) {

@@ -29,7 +29,14 @@ two of 1.5 ff), layers latent - delta - delta - attention against attention - li
 see a window of 1024 tokens and are priced on the keys they see; its latent attention reads [latent ; rotated part] once per key (the
 values are a view of the keys); the delta rule is priced like the lightning recurrence — prompts on the multiply-adds of the recurrence
 (three products of a dim x vdim state per token and head), decode rows on the state bytes read and written.
+
+Sabezen (`--lm-model sabezen`) also stands beside Zuzenex — the same step function, parallel layers that choose attention or a matrix-state
+recurrence — and its delta rule beside Daberax's: same width, depth, head counts and 128-wide heads, layers attention - channel delta -
+gla - attention, once with dense feed-forwards of equal size (two matrices of 1.5 ff on both), once with 8 experts top-2 on both (three
+matrices of ff / 2; no shared expert).  Its attention sees chunks of 1024 tokens and is priced on the pairs it sees; the mixing of the
+heads' scores is not counted as work.  The recurrences are priced like the lightning recurrence and the delta rule.
 """
+import sys
 import time
 
 import torch
@@ -434,6 +441,124 @@ def run_daberax(s, T, batches, n_dec, window=1024):
     return out
 
 
+SABEZEN_CHUNK = 1024
+
+
+def sabezen_config(s, dense=True, chunk=SABEZEN_CHUNK):
+    from .configuration import SabezenConfig
+    H = s["heads"]
+    mlp = dict(kind="dense", ff=s["ff"] * 3 // 2) if dense else dict(kind="moe", router=dict(experts=8, top=2), expert=dict(ff=s["ff"] // 2))
+    att = dict(type="attention", mixer=dict(heads=H, kv_heads=H // 4, dim=128, vdim=128, scale=128 ** -0.5, rot=dict(base=100000.0, dims=64),
+                                            mask=dict(size=chunk)), mlp=mlp)
+    dlt = dict(type="channel_delta", mixer=dict(heads=H, kv_heads=H, dim=128, vdim=128, conv=4), mlp=mlp)
+    gla = dict(type="gla", mixer=dict(heads=H, dim=128, vdim=128, tau=16.0), mlp=mlp)
+    order = [att, dlt, gla, att]
+    return SabezenConfig(width=s["width"], vocab=s["vocab"], layers=[order[i % 4] for i in range(s["layers"])], norm=dict(eps=1e-6),
+                         embedding=dict(scale=2.0))
+
+
+def run_sabezen(s, T, batches, n_dec, dense=True, kernels=True):
+    from ._lib import LowRankJob, check, current_stream, lib, ptr
+    from .sabezen import SabezenDecoder
+    from .sequences import rows_of_spans
+    dev = "cuda"
+    dec = SabezenDecoder.synthetic(sabezen_config(s, dense), dev, t_max=T + n_dec + 8, n_seq=max(batches), arith="bf16")
+    ids = torch.randint(0, s["vocab"], (T,), device=dev)
+    x = dec.embed(ids)
+    out = {"prefill_tokens_per_s": T / _time(lambda: dec.forward_spans(x, [(0, T, 0)], tokens=ids), 3)}
+    for B in batches:
+        for ly in dec.state_t:                               # every sequence continues the prompt of sequence 0
+            for t in ly.values():
+                if t is not None and B > 1:
+                    t[1:B].copy_(t[0:1].expand_as(t[1:B]))
+        row_seq = torch.arange(B, dtype=torch.int32, device=dev)
+        back, blk = dec.decode_tables(B)
+        tok = torch.randint(0, s["vocab"], (B,), device=dev)
+        xb, tok32 = dec.embed(tok), tok.to(torch.int32)
+        more = dict(row_tok=tok32) if dec.needs_tokens else {}
+
+        def loop():
+            slot = torch.full((B,), T, dtype=torch.int32, device=dev)
+            ln = slot + 1
+            for i in range(n_dec):
+                dec.step(xb, row_seq, slot, back, ln, blk, T + i + 1, distinct=True, **more)
+                check(lib().mn_rows_advance(ptr(slot), ptr(ln), None, B, 1, current_stream()), "mn_rows_advance")
+        out[f"decode_b{B}_tokens_per_s"] = B * n_dec / _time(loop, 2, 1)
+        slot_g = torch.full((B,), T, dtype=torch.int32, device=dev)
+        ln_g = slot_g + 1
+        graph = dec.decode_graph(row_seq, slot_g, ln_g)
+
+        def loop_graph():
+            slot_g.fill_(T)
+            ln_g.fill_(T + 1)
+            for i in range(n_dec):
+                graph.run(xb, T + i + 1, tokens=tok32)
+        out[f"decode_b{B}_graph_tokens_per_s"] = B * n_dec / _time(loop_graph, 2, 1)
+    if not kernels:
+        return out
+    # the kernels alone, on the layers' own arenas and states
+    H, G, d, chunk = s["heads"], s["heads"] // 4, 128, SABEZEN_CHUNK
+    RB = dec.block_rows
+    tabs = {k: torch.from_numpy(v).to(dev) for k, v in rows_of_spans([(0, T, 0)], RB, dec.chunk_rows).items() if k != "max_len"}
+    st = dec.state_t[0]
+    q, att = torch.randn(T, H * d, device=dev) * 0.05, torch.empty(T, H * d, device=dev)
+    talk, sink = torch.eye(H, device=dev) + 0.1 * torch.randn(H, H, device=dev), torch.zeros(H, device=dev)
+    aws = torch.empty(128 << 20, dtype=torch.uint8, device=dev)
+
+    def attn(M, rs, rp, one_row):
+        n_blk, rows = (M, 1) if one_row else (tabs["blk_tab"].shape[0], RB)
+        ns = lib().mn_talk_attn_splits(n_blk, chunk)
+        check(lib().mn_talk_attn(ptr(q), H * d, ptr(st["k"]), G * d, ptr(st["v"]), G * d, ptr(talk), ptr(sink), ptr(rs), ptr(rp), M,
+                                 None if one_row else ptr(tabs["blk_tab"]), n_blk, rows, H, G, d, dec.t_max, 0, chunk, ptr(att), H * d, None, 0,
+                                 ns, ptr(aws), aws.numel(), -1, current_stream()), "mn_talk_attn")
+        return ns
+    t = _time(lambda: attn(T, tabs["row_seq"], tabs["row_slot"], 0), 5)
+    flops = 2 * 2 * H * d * sum(i % chunk + 1 for i in range(T))
+    out["attn_prefill"] = dict(us=t * 1e6, tflops=flops / t / 1e12, of_peak=flops / t / 1e12 / FMA_F32_TFLOPS, peak="fp32 MFMA",
+                               key_splits=attn(T, tabs["row_seq"], tabs["row_slot"], 0))
+    for B in batches:
+        row_seq = torch.arange(B, dtype=torch.int32, device=dev)
+        slot = torch.full((B,), T - 1, dtype=torch.int32, device=dev)
+        t = _time(lambda: attn(B, row_seq, slot, 1), 20)
+        byts = B * ((T - 1) % chunk + 1) * G * 2 * d * 4
+        out[f"attn_decode_b{B}"] = dict(us=t * 1e6, gbs=byts / t / 1e9, of_peak=byts / t / 1e9 / HBM_GBS, key_splits=attn(B, row_seq, slot, 1))
+    # the two recurrences alone
+    qkv, o = torch.randn(T, 3 * H * d, device=dev), torch.empty(T, H * d, device=dev)
+    qkv[:, :2 * H * d] *= d ** -0.5
+    g, beta = 0.9 + 0.1 * torch.rand(T, H * d, device=dev), torch.rand(T, H, device=dev)
+    for name, li, b in (("delta", 1, beta), ("gla", 2, None)):
+        lin = dec.state_t[li]["lin"]
+
+        def state_rows(M, rs, rp, rb, flags):
+            check(lib().mn_channel_state_rows(ptr(qkv), 3 * H * d, ptr(g), H * d, ptr(b), H, M, H, H, d, d, 1.0, ptr(lin), ptr(rs), ptr(rp), ptr(rb),
+                                              None if flags else ptr(tabs["blk_tab"]), 0 if flags else tabs["blk_tab"].shape[0], flags, ptr(o),
+                                              H * d, current_stream()), "mn_channel_state_rows")
+        n_ch = tabs["chunk_tab"].shape[0]
+
+        def scan():
+            check(lib().mn_channel_state_rows_scan(ptr(qkv), 3 * H * d, ptr(g), H * d, T, H, H, d, d, 1.0, ptr(lin), ptr(tabs["row_seq"]),
+                                                   ptr(tabs["row_slot"]), ptr(tabs["row_back"]), ptr(tabs["chunk_tab"]), n_ch, ptr(o), H * d,
+                                                   ptr(aws), aws.numel(), current_stream()), "mn_channel_state_rows_scan")
+        t = _time(scan if b is None else (lambda: state_rows(T, tabs["row_seq"], tabs["row_slot"], tabs["row_back"], 0)), 5)
+        flops = 2 * T * H * (3 if b is not None else 2) * d * d
+        out[name + "_prefill"] = dict(us=t * 1e6, tflops=flops / t / 1e12, of_peak=flops / t / 1e12 / FMA_F32_TFLOPS, peak="fp32 FMA")
+        for B in batches:
+            row_seq = torch.arange(B, dtype=torch.int32, device=dev)
+            slot = torch.full((B,), T - 1, dtype=torch.int32, device=dev)
+            t = _time(lambda: state_rows(B, row_seq, slot, None, 1), 20)
+            byts = B * H * d * d * 4 * 2
+            out[f"{name}_decode_b{B}"] = dict(us=t * 1e6, gbs=byts / t / 1e9, of_peak=byts / t / 1e9 / HBM_GBS)
+    # the low-rank decays and gates of a prompt (two products of rank 128 with the gate functions behind them)
+    a1, w2 = torch.randn(T, 256, device=dev), torch.randn(H * d, 128, device=dev).to(torch.bfloat16)
+    a_log, dts = torch.zeros(H, device=dev), torch.zeros(H * d, device=dev, dtype=torch.bfloat16)
+    jobs = (LowRankJob * 2)(LowRankJob(a1.data_ptr(), 256, w2.data_ptr(), dts.data_ptr(), a_log.data_ptr(), g.data_ptr(), H * d, 128, H * d, 1, d, 1.0),
+                            LowRankJob(a1.data_ptr() + 512, 256, w2.data_ptr(), None, None, o.data_ptr(), H * d, 128, H * d, 3, 1, 1.0))
+    t = _time(lambda: check(lib().mn_low_rank_gate_rows(jobs, 2, T, current_stream()), "mn_low_rank_gate_rows"), 5)
+    flops = 2 * 2 * T * H * d * 128
+    out["low_rank_prefill"] = dict(us=t * 1e6, tflops=flops / t / 1e12, of_peak=flops / t / 1e12 / FMA_F32_TFLOPS, peak="fp32 MFMA")
+    return out
+
+
 def run_bailing(s, T, batches, n_dec, shared=0):
     from . import ops
     from ._lib import check, current_stream, lib, ptr
@@ -483,6 +608,16 @@ def compare(sizes=("w1024", "w2048"), prompt=2048, batches=(1, 32), n_dec=32, mo
     for name in sizes:
         s = SIZES[name]
         torch.cuda.empty_cache()
+        if model == "sabezen":                               # beside the models with the like kernels, with dense and with expert feed-forwards
+            res[name] = dict(size=s, prompt=prompt)
+            for key, run in (("sabezen_dense", lambda: run_sabezen(s, prompt, batches, n_dec)),
+                             ("zuzenex_dense", lambda: run_zuzenex(s, prompt, batches, n_dec, dense=True)),
+                             ("sabezen_moe", lambda: run_sabezen(s, prompt, batches, n_dec, dense=False, kernels=False)),
+                             ("zuzenex_moe", lambda: run_zuzenex(s, prompt, batches, n_dec)), ("daberax", lambda: run_daberax(s, prompt, batches, n_dec))):
+                res[name][key] = run()
+                torch.cuda.empty_cache()
+                print(f"[lm-compare] {name} {key}", file=sys.stderr, flush=True)
+            continue
         if model == "daberax":                               # beside the closest model of the framework instead of the Bailing-MoE decoder
             res[name] = dict(size=s, prompt=prompt, daberax=run_daberax(s, prompt, batches, n_dec))
             torch.cuda.empty_cache()

@@ -134,6 +134,8 @@ class SabezenDecoder(HybridSteps, SeqDecoder):
         # rows per run of the attention: what every attention layer's matrix-core kernel takes (a layer without an instance takes any)
         takes = [lib().mn_talk_attn_block_rows(L.heads, L.kv_heads, L.dim) for L in layers if L.kind == KIND["attention"]]
         self.block_rows = min([int(r) for r in takes if r > 0] or [8])
+        if any(L.kind == KIND["gla"] for L in layers):
+            self.chunk_rows = int(lib().mn_channel_chunk_rows())
         s = HybModel()
         s.width, s.n_layers, s.n_runs, s.arith, s.eps = W, n, n, ARITH[arith], cfg.eps
         s.norm, s.vocab, s.block_rows = NORM_LAYER, cfg.vocab, self.block_rows
