@@ -366,7 +366,6 @@ __global__ __launch_bounds__(256) void delta_rows_fast_kernel(DeltaArgs a) {
     const int i = 4 * (s + LPC * (j >> 2)) + (j & 3);
     S[j] = (on && !fresh && i < d) ? sp[(int64_t)i * a.vdim] : 0.f;
   }
-  __syncthreads();                           // the state has arrived: from here on only a batch's loads are in flight
   float* qk = lds;                           // row r: q at r * 2 DP, k at r * 2 DP + DP
   float* vs = qk + DBT * 2 * DP;
   float* bs = vs + DBT * CPB;
