@@ -28,7 +28,7 @@
 extern "C" {
 #endif
 
-#define MN_VERSION 130 /* 0.1.30: layers with a decay per key channel and mixed attention heads (section 13).  0.1.29: post-norm mixed-mixer sequence models (section 12).  0.1.28: hybrid-mixer sequence models (section 11).  0.1.27: parallel-mixer sequence models (section 10).  0.1.26: latent-cache sequence models (section 9).  0.1.24: mn_persist_set_status_word; mn_tp_allreduce PUSH|REDUCE above the one-shot row limit implies GATHER.  0.1.23: ABI guards mn_sizeof_* / mn_struct_layout.  0.1.20: fp8 weight mode (section 7): wfmt / row-scale fields at the END of mn_skinny_args, mn_rf_head,
+#define MN_VERSION 131 /* 0.1.31: multi-stream sequence models (section 14).  0.1.30: layers with a decay per key channel and mixed attention heads (section 13).  0.1.29: post-norm mixed-mixer sequence models (section 12).  0.1.28: hybrid-mixer sequence models (section 11).  0.1.27: parallel-mixer sequence models (section 10).  0.1.26: latent-cache sequence models (section 9).  0.1.24: mn_persist_set_status_word; mn_tp_allreduce PUSH|REDUCE above the one-shot row limit implies GATHER.  0.1.23: ABI guards mn_sizeof_* / mn_struct_layout.  0.1.20: fp8 weight mode (section 7): wfmt / row-scale fields at the END of mn_skinny_args, mn_rf_head,
                           mn_llm and mn_llm_tp (zero = bf16: callers of 0.1.10 that zero-fill the structs are unchanged),
                           mn_quant_fp8_rows / mn_dequant_fp8_rows / mn_stream_mfma_w8 / mn_stream_mfma_grouped_w8 */
 
@@ -1403,6 +1403,108 @@ MN_API int mn_talk_attn(const float* q, int64_t ldq, const float* k_arena, int64
                         const float* sink, const int32_t* row_seq, const int32_t* row_slot, int M, const int32_t* blk_tab, int n_blk, int rows,
                         int H, int G, int dim, int t_max, int window, int chunk, float* out, int64_t ldo, uint16_t* out16, int64_t ldo16,
                         int nsplit, void* workspace, size_t workspace_bytes, int variant, void* stream);
+
+/* ------------------------------------------------------------------------------------------
+ * 14. Multi-stream sequence models (0.1.31): decoder stacks whose residual is S parallel streams of the model's width.  A sublayer reads
+ *     u = sum_s in[s] x_s and norms it; its result y goes back as x_t <- sum_s mix[s, t] x_s + out[t] y, all streams at once from the old
+ *     ones (mix is indexed [from, to]).  Sublayers run one after the other: softmax attention (biases, RMS norm over the whole q and k
+ *     projections, rotary pairs, chunk and / or window, sinks, values mixed with those of the first mixing layer, an output gate per
+ *     value), then a mixture of silu-gated experts with a sigmoid router whose scores scale the experts' INPUT.  Streams, norms, angles,
+ *     scores, softmax, router and cached keys / values are fp32 in both arithmetic modes.
+ * ------------------------------------------------------------------------------------------ */
+/* One launch between two sublayers, per row m: y = y[m] (optional) + sum_j ew_j ye[r(m, j)] (top > 0; r as in mn_moe_combine_residual, ew NULL:
+ * every weight 1); with mix: x_t <- sum_s mix[s, t] x_s + out[t] y, stored to dst when given (in place allowed: dst = src); then
+ * u = sum_s in[s] x_s (in NULL: the streams' sum) and, with w, u / sqrt(mean(u^2) + eps) * w (one_plus: * (1 + w)), to h (fp32) and / or
+ * h16 (bf16).  Stream s of row m starts at src + m src_row + s src_stream (src_stream 0: all streams are the same row). */
+typedef struct mn_streams_args {
+  const float* src; int64_t src_row, src_stream;
+  float* dst;                                      /* [M, S, n] or NULL */
+  int32_t S, n;
+  const float *mix, *out, *in;                     /* DEVICE fp32 [S, S], [S], [S] */
+  const float* y; int64_t ldy;
+  const float* ye; int64_t ldye;
+  const int32_t* slot_of; const float* ew;
+  int32_t top, one_plus;
+  const uint16_t* w;                               /* [n] or NULL: no norm */
+  float eps;
+  float* h; int64_t ldh;
+  uint16_t* h16; int64_t ldh16;
+} mn_streams_args;
+MN_API size_t mn_sizeof_streams_args(void);
+MN_API int mn_streams_update_norm(const mn_streams_args* a, int M, void* stream);
+/* mn_proj_norm_rope_append with cos and sin multiplied by rot_mag, and with values that are mixed: v_keep (optional, fp32 [M, kv_heads vdim])
+ * receives the row's values as projected; v_first (optional): v <- (1 - v_lambda) v + v_lambda v_first before the append. */
+MN_API int mn_proj_norm_rope_mix_append(const float* qkv, int64_t ldqkv, int M, int H, int G, int dim, int vdim, const uint16_t* q_norm,
+                                        const uint16_t* k_norm, float eps, int rot_dims, int interleaved, const float* freq, float rot_mag,
+                                        float q_scale, float* v_keep, int64_t ldvk, const float* v_first, int64_t ldvf, float v_lambda,
+                                        const int32_t* row_seq, const int32_t* row_slot, float* q_out, int64_t ldq, float* k_arena,
+                                        int64_t ldk, float* v_arena, int64_t ldv, int t_max, void* stream);
+/* mn_window_pool_attn_blocks_cap with chunks (chunk > 0: position i sees j <= i only if floor(i / chunk) = floor(j / chunk), positions counted
+ * from the sequence's start; not together with pooled blocks) and a gate (fp32 [M, H vdim] or NULL): every result times sigmoid(its gate). */
+MN_API int mn_window_pool_attn_blocks_gate(const float* q, int64_t ldq, const float* k_arena, int64_t ldk, const float* v_arena, int64_t ldv,
+                                           const float* pk, const float* pv, const float* sink, float softcap, int chunk, const float* gate,
+                                           int64_t ldgate, const int32_t* row_seq, const int32_t* row_slot, const int32_t* blk_tab, int n_blk,
+                                           int one_row, int H, int G, int dim, int vdim, int t_max, int n_pool_max, int window, int pool,
+                                           float out_scale, float* out, int64_t ldo, uint16_t* out16, int64_t ldo16, int nsplit, void* workspace,
+                                           size_t workspace_bytes, int variant, void* stream);
+/* The `top` largest of logits[m, 0 .. E) (ties: the lower index) and their sigmoids as they are: idx int32 [M, top], w fp32 [M, top] */
+MN_API int mn_router_sigmoid_topk_rows(const float* logits, int64_t ld, int M, int E, int top, int32_t* idx, float* w, void* stream);
+/* Experts that are fed with weight * input: the weight is a factor of the gate and up products.
+ * mn_moe_sort_weights: mn_moe_sort (tile_g NULL) or mn_moe_sort_tiles; w_sorted[slot_of[z]] = topk_w[z].
+ * *_scaled: silu(s gate) * (s up) with a factor s per row / pair (row_scale, x_scale; NULL: 1; the grouped GEMM: epi 6 only, by position). */
+MN_API int mn_moe_sort_weights(const int32_t* topk_idx, const float* topk_w, int T, int n_slot, int n_groups, int32_t* counts, int32_t* offsets,
+                               int32_t* perm, int32_t* slot_of, float* w_sorted, int tile_rows, int32_t* tile_g, int32_t* tile_m0,
+                               int32_t* n_tiles, void* stream);
+MN_API int mn_gemm256_grouped_tiles_scaled(const uint16_t* A, int64_t lda, int64_t a_lo_off, int64_t a_rows_total, const int32_t* a_rows,
+                                           const uint16_t* W, int64_t ldw, int64_t w_gstride, const int32_t* off, const int32_t* cnt,
+                                           int n_groups, const int32_t* tile_g, const int32_t* tile_m0, const int32_t* n_tiles, int max_mtiles,
+                                           const float* row_scale, void* C, int64_t ldc, int64_t c_lo_off, int N, int K, int epi, void* stream);
+MN_API int mn_silu_mul_rows_scaled(const float* x, int64_t ldx, const float* x_scale, float* y, int64_t ldy, uint16_t* y16, int64_t ldy16, int M,
+                                   int n, void* stream);
+MN_API int mn_gemv_glu_indexed_scaled(const float* A, int64_t lda, int a_div, const uint16_t* W, int64_t ldw, int64_t w_bs, const int32_t* w_idx,
+                                      int n_idx, const float* x_scale, float* C, int64_t ldc, int Z, int N, int K, void* stream);
+
+typedef struct mn_ms_layer {
+  int32_t heads, kv_heads, dim, vdim;
+  int32_t rot_dims, rot_interleaved;               /* values of a head that turn; 0: none */
+  int32_t window, chunk;                           /* 0: none */
+  int32_t has_gate;                                /* 1 = a gate per value follows v in the stack */
+  int32_t v_mix;                                   /* 1: the first such layer's values are mixed into the later ones' */
+  int32_t experts, top, expert_ff;                 /* experts 0: no feed-forward */
+  float scale, rot_mag, v_lambda;
+  const float* rot_freq;                           /* DEVICE fp32 [rot_dims / 2] */
+  const float* sink;                               /* DEVICE fp32 [heads] or NULL: exp(sink[h]) joins the softmax's denominator */
+  const float *hc1_in, *hc1_out, *hc1_mix;         /* DEVICE fp32 [streams], [streams], [streams, streams] = [from, to] */
+  const float *hc2_in, *hc2_out, *hc2_mix;
+  const uint16_t *norm1, *norm2;                   /* [width] */
+  const uint16_t *w_in, *b_in;                     /* [q ; k ; v ; gate], zero rows up to a multiple of 8; bias or NULL */
+  const uint16_t *q_norm, *k_norm;                 /* [heads dim], [kv_heads dim] or NULL */
+  const uint16_t* w_o;                             /* [width, heads vdim] */
+  const uint16_t* w_router;                        /* [experts rounded up to a multiple of 8, width] */
+  const uint16_t* w_gate_up;                       /* [experts, 2 expert_ff, width] = [gate ; up] */
+  const uint16_t* w_down;                          /* [experts, width, expert_ff] */
+} mn_ms_layer;
+typedef struct mn_ms_model {
+  int32_t width, n_layers, streams, arith;
+  int32_t norm_one_plus;                           /* 1: the layers' and the final norm's weights are stored around zero */
+  float eps;
+  const mn_ms_layer* layers;                       /* HOST array [n_layers] */
+  const uint16_t* final_w;
+} mn_ms_model;
+typedef struct mn_ms_state {                       /* HOST arrays [n_layers] of device pointers, fp32 */
+  float* const* k;                                 /* [n_seq, t_max, kv_heads dim] */
+  float* const* v;                                 /* [n_seq, t_max, kv_heads vdim], mixed */
+  int32_t n_seq, t_max;
+} mn_ms_state;
+MN_API size_t mn_sizeof_ms_layer(void);
+MN_API size_t mn_sizeof_ms_model(void);
+MN_API size_t mn_sizeof_ms_state(void);
+/* One pass of the stack over M rows; rows, row arrays, blk_tab / n_blk, max_len, flags, out and trace as mn_pmix_step (trace: fp32
+ * [n_layers, M, width], the streams' sum after every layer). */
+MN_API size_t mn_ms_workspace_bytes(const mn_ms_model* m, int M);
+MN_API int mn_ms_step(const mn_ms_model* m, const mn_ms_state* st, const float* x, int64_t ldx, int M, const int32_t* row_seq,
+                      const int32_t* row_slot, const int32_t* blk_tab, int n_blk, int max_len, int flags, float* out, float* trace,
+                      void* workspace, size_t workspace_bytes, void* stream);
 
 #ifdef __cplusplus
 }

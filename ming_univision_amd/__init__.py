@@ -47,6 +47,9 @@ def __getattr__(name):  # lazy: keep `import ming_univision_amd` cheap and torch
     if name in ("SabezenDecoder", "SabezenForCausalLM"):
         from . import sabezen
         return getattr(sabezen, name)
+    if name in ("FegaraxDecoder", "FegaraxForCausalLM"):
+        from . import fegarax
+        return getattr(fegarax, name)
     if name == "load_model":
         from .infer import load_model
         return load_model

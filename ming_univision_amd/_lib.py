@@ -192,6 +192,30 @@ class PnState(C.Structure):
     _fields_ = [(k, PP) for k in ("k", "v", "conv", "lin")] + [("n_seq", C.c_int32), ("t_max", C.c_int32)]
 
 
+class StreamsArgs(C.Structure):
+    _fields_ = [("src", C.c_void_p), ("src_row", C.c_int64), ("src_stream", C.c_int64), ("dst", C.c_void_p), ("S", C.c_int32), ("n", C.c_int32),
+                ("mix", C.c_void_p), ("out", C.c_void_p), ("in_", C.c_void_p), ("y", C.c_void_p), ("ldy", C.c_int64), ("ye", C.c_void_p),
+                ("ldye", C.c_int64), ("slot_of", C.c_void_p), ("ew", C.c_void_p), ("top", C.c_int32), ("one_plus", C.c_int32),
+                ("w", C.c_void_p), ("eps", C.c_float), ("h", C.c_void_p), ("ldh", C.c_int64), ("h16", C.c_void_p), ("ldh16", C.c_int64)]
+
+
+class MsLayer(C.Structure):
+    _fields_ = [(k, C.c_int32) for k in ("heads", "kv_heads", "dim", "vdim", "rot_dims", "rot_interleaved", "window", "chunk", "has_gate", "v_mix",
+                                         "experts", "top", "expert_ff")] + \
+               [(k, C.c_float) for k in ("scale", "rot_mag", "v_lambda")] + \
+               [(k, C.c_void_p) for k in ("rot_freq", "sink", "hc1_in", "hc1_out", "hc1_mix", "hc2_in", "hc2_out", "hc2_mix", "norm1", "norm2",
+                                          "w_in", "b_in", "q_norm", "k_norm", "w_o", "w_router", "w_gate_up", "w_down")]
+
+
+class MsModel(C.Structure):
+    _fields_ = [(k, C.c_int32) for k in ("width", "n_layers", "streams", "arith", "norm_one_plus")] + \
+               [("eps", C.c_float), ("layers", C.POINTER(MsLayer)), ("final_w", C.c_void_p)]
+
+
+class MsState(C.Structure):
+    _fields_ = [(k, PP) for k in ("k", "v")] + [("n_seq", C.c_int32), ("t_max", C.c_int32)]
+
+
 # (struct id of mn_struct_layout, its mn_sizeof_* export, the ctypes mirror): checked against the library at load time (`lib()`)
 STRUCTS = ((0, "mn_sizeof_skinny_args", SkinnyArgs), (1, "mn_sizeof_rf_head", RfHead), (2, "mn_sizeof_llm", Llm),
            (3, "mn_sizeof_semdec", SemDec), (4, "mn_sizeof_tp_comm", TpComm), (5, "mn_sizeof_llm_tp", LlmTp),
@@ -199,7 +223,9 @@ STRUCTS = ((0, "mn_sizeof_skinny_args", SkinnyArgs), (1, "mn_sizeof_rf_head", Rf
            (9, "mn_sizeof_pmix_layer", PmixLayer), (10, "mn_sizeof_pmix_model", PmixModel), (11, "mn_sizeof_pmix_state", PmixState),
            (12, "mn_sizeof_hyb_layer", HybLayer), (13, "mn_sizeof_hyb_model", HybModel), (14, "mn_sizeof_hyb_state", HybState),
            (15, "mn_sizeof_pn_layer", PnLayer), (16, "mn_sizeof_pn_model", PnModel), (17, "mn_sizeof_pn_state", PnState),
-           (18, "mn_sizeof_low_rank_job", LowRankJob), (19, "mn_sizeof_rows_prep", RowsPrep))
+           (18, "mn_sizeof_low_rank_job", LowRankJob), (19, "mn_sizeof_rows_prep", RowsPrep),
+           (20, "mn_sizeof_streams_args", StreamsArgs), (21, "mn_sizeof_ms_layer", MsLayer), (22, "mn_sizeof_ms_model", MsModel),
+           (23, "mn_sizeof_ms_state", MsState))
 
 
 def check_struct_layouts(handle):
@@ -441,6 +467,20 @@ SYMBOLS = {
     "mn_talk_attn_workspace_bytes": (_sz, [_i, _i, _i, _i, _i, _i]),
     "mn_talk_attn": (_i, [_p, _i64, _p, _i64, _p, _i64, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p, _i64, _p, _i64, _i, _p, _sz,
                           _i, _p]),
+    # section 14: multi-stream sequence models
+    "mn_sizeof_streams_args": (_sz, []), "mn_sizeof_ms_layer": (_sz, []), "mn_sizeof_ms_model": (_sz, []), "mn_sizeof_ms_state": (_sz, []),
+    "mn_streams_update_norm": (_i, [C.POINTER(StreamsArgs), _i, _p]),
+    "mn_proj_norm_rope_mix_append": (_i, [_p, _i64, _i, _i, _i, _i, _i, _p, _p, _f, _i, _i, _p, _f, _f, _p, _i64, _p, _i64, _f, _p, _p, _p, _i64, _p,
+                                          _i64, _p, _i64, _i, _p]),
+    "mn_window_pool_attn_blocks_gate": (_i, [_p, _i64, _p, _i64, _p, _i64, _p, _p, _p, _f, _i, _p, _i64, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i,
+                                             _i, _i, _f, _p, _i64, _p, _i64, _i, _p, _sz, _i, _p]),
+    "mn_router_sigmoid_topk_rows": (_i, [_p, _i64, _i, _i, _i, _p, _p, _p]),
+    "mn_moe_sort_weights": (_i, [_p, _p, _i, _i, _i, _p, _p, _p, _p, _p, _i, _p, _p, _p, _p]),
+    "mn_gemm256_grouped_tiles_scaled": (_i, [_p, _i64, _i64, _i64, _p, _p, _i64, _i64, _p, _p, _i, _p, _p, _p, _i, _p, _p, _i64, _i64, _i, _i, _i, _p]),
+    "mn_silu_mul_rows_scaled": (_i, [_p, _i64, _p, _p, _i64, _p, _i64, _i, _i, _p]),
+    "mn_gemv_glu_indexed_scaled": (_i, [_p, _i64, _i, _p, _i64, _i64, _p, _i, _p, _p, _i64, _i, _i, _i, _p]),
+    "mn_ms_workspace_bytes": (_sz, [C.POINTER(MsModel), _i]),
+    "mn_ms_step": (_i, [C.POINTER(MsModel), C.POINTER(MsState), _p, _i64, _i, _p, _p, _p, _i, _i, _i, _p, _p, _p, _sz, _p]),
     "mn_semdec_step": (_i, [C.POINTER(SemDec), _p, _i, _p, _p, _p, _p, _i, _i64, _p, _p, _p, _sz, _p]),
 }
 
@@ -461,7 +501,7 @@ def lib():
         fn = getattr(handle, name)  # AttributeError if the symbol is missing
         fn.restype = res
         fn.argtypes = args
-    if handle.mn_version() < 130:
+    if handle.mn_version() < 131:
         raise RuntimeError("libmingnative.so is too old")
     check_struct_layouts(handle)
     _lib = handle

@@ -807,6 +807,95 @@ def sabezen_param_shapes(cfg: SabezenConfig, ranks):
     return s
 
 
+# ---- Fegarax ---------------------------------------------------------------------------------------------------------------
+class FegaraxConfig(_Config):
+    """A stack of pre-norm layers over several residual streams.  `layers` is a list of dicts(type, mixer, mlp):
+    type "attention": mixer dict(heads, kv_heads, dim, vdim, scale, optional rot dict(base, dims, optional scaling dict(factor, original, fast,
+          slow)), optional mask dict(size), optional v_mix): biases, RMS norm over the whole q and k projections, rotary half pairs, chunks of
+          mask.size positions that see only themselves, one added to the softmax's denominator, values mixed with those of the first
+          v_mix layer, an output gate per value
+    mlp   None or dict(kind="moe", router dict(experts, top), expert dict(ff)): silu-gated experts, sigmoid scores that scale their input
+    streams: residual streams (None: one, added to as it is); embedding dict(scale): factor of the input embeddings, whose table is also
+    the vocabulary projection.  Nothing is assumed equal between layers."""
+    model_type = "fegarax"
+
+    def __init__(self, width=256, vocab=1024, layers=(), norm=None, embedding=None, streams=None, architecture="Fegarax", **kwargs):
+        self.architecture = architecture
+        self.width, self.vocab = int(width), int(vocab)
+        self.layers = [copy.deepcopy(dict(ly)) for ly in layers]
+        self.norm = dict(norm or {"eps": 1e-6})
+        self.embedding = dict(embedding or {})
+        self.streams = None if streams is None else int(streams)
+        super().__init__(**kwargs)
+        self.validate()
+
+    eps = property(lambda self: float(self.norm["eps"]))
+    embed_scale = property(lambda self: float(self.embedding.get("scale", 1.0)))
+
+    def validate(self):
+        if self.streams is not None and self.streams < 1:
+            raise ValueError(f"streams = {self.streams} must be >= 1")
+        mixed = None
+        for i, ly in enumerate(self.layers):
+            if ly.get("type") != "attention":
+                raise ValueError(f"layer {i}: unknown mixer type {ly.get('type')!r} (known: 'attention')")
+            m = ly["mixer"]
+            for k in ("heads", "kv_heads", "dim", "vdim", "scale"):
+                if k not in m:
+                    raise ValueError(f"layer {i}: mixer lacks {k!r}")
+            if int(m["heads"]) % int(m["kv_heads"]):
+                raise ValueError(f"layer {i}: {m['heads']} heads do not divide over {m['kv_heads']} key heads")
+            rot = m.get("rot")
+            if rot and (int(rot["dims"]) % 2 or not (0 <= int(rot["dims"]) <= int(m["dim"]))):
+                raise ValueError(f"layer {i}: rot.dims = {rot['dims']} must be even and at most {m['dim']}")
+            sc = rot.get("scaling") if rot else None
+            if sc and not all(float(sc[k]) > 0 for k in ("factor", "original", "fast", "slow")):
+                raise ValueError(f"layer {i}: rot.scaling {sc}: factor, original, fast and slow must be positive")
+            if m.get("mask") and int(m["mask"]["size"]) < 1:
+                raise ValueError(f"layer {i}: mask.size must be >= 1")
+            if m.get("v_mix"):
+                n = int(m["kv_heads"]) * int(m["vdim"])
+                mixed = mixed or n
+                if n != mixed:
+                    raise ValueError(f"layer {i}: its {n} values do not mix with the {mixed} of the first v_mix layer")
+            mlp = ly.get("mlp")
+            if mlp is None:
+                continue
+            if mlp.get("kind") != "moe":
+                raise ValueError(f"layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
+            r = mlp["router"]
+            if not (1 <= int(r["top"]) <= int(r["experts"])) or int(mlp["expert"]["ff"]) < 1:
+                raise ValueError(f"layer {i}: router {r}: 1 <= top <= experts, and expert.ff >= 1")
+
+
+def fegarax_param_shapes(cfg: FegaraxConfig):
+    """{tensor name: shape} of a Fegarax checkpoint (`l<i>.` per layer, `mix.` the mixer's, `mlp.` the experts' and `hc1.` / `hc2.` the stream
+    mixing's tensors of its two sublayers)."""
+    W, V, S = cfg.width, cfg.vocab, cfg.streams
+    s = {"embed": (V, W)}
+    for i, ly in enumerate(cfg.layers):
+        p, m, mlp = f"l{i}.", ly["mixer"], ly.get("mlp")
+        H, G, d, e = int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"])
+        s[p + "norm1"] = (W,)
+        for n, rows in (("q", H * d), ("k", G * d), ("v", G * e)):
+            s[p + "mix." + n], s[p + "mix." + n + ".b"] = (rows, W), (rows,)
+        s[p + "mix.q.norm"], s[p + "mix.k.norm"] = (H * d,), (G * d,)
+        if m.get("v_mix"):
+            s[p + "mix.vmix"] = ()
+        s[p + "mix.g"], s[p + "mix.o"] = (H * e, W), (W, H * e)
+        if mlp is not None:
+            E, ff = int(mlp["router"]["experts"]), int(mlp["expert"]["ff"])
+            s[p + "norm2"] = (W,)
+            for j in range(E):
+                s[f"{p}mlp.e{j}.gate"], s[f"{p}mlp.e{j}.up"], s[f"{p}mlp.e{j}.down"] = (ff, W), (ff, W), (W, ff)
+            s[p + "mlp.router"] = (E, W)
+        for q in (1, 2) if mlp is not None else (1,):
+            if S is not None:
+                s[f"{p}hc{q}.in"], s[f"{p}hc{q}.out"], s[f"{p}hc{q}.mix"] = (S,), (S,), (S, S)
+    s["final.norm"] = (W,)
+    return s
+
+
 # ---- registry: which configuration class a config.json belongs to -------------------------------------------------------------
 def _is_pizitar(d):
     return d.get("architecture") == "Pizitar" or d.get("model_type") == "pizitar"
@@ -828,12 +917,16 @@ def _is_sabezen(d):
     return d.get("architecture") == "Sabezen" or d.get("model_type") == "sabezen"
 
 
+def _is_fegarax(d):
+    return d.get("architecture") == "Fegarax" or d.get("model_type") == "fegarax"
+
+
 def _is_ming_univision(d):
     return "llm_config" in d or d.get("model_type") in ("bailingmm", "ming_univision")
 
 
 MODEL_REGISTRY = [("pizitar", _is_pizitar, PizitarConfig), ("sakinex", _is_sakinex, SakinexConfig), ("zuzenex", _is_zuzenex, ZuzenexConfig),
-                  ("daberax", _is_daberax, DaberaxConfig), ("sabezen", _is_sabezen, SabezenConfig),
+                  ("daberax", _is_daberax, DaberaxConfig), ("sabezen", _is_sabezen, SabezenConfig), ("fegarax", _is_fegarax, FegaraxConfig),
                   ("ming_univision", _is_ming_univision, MingUniVisionConfig)]
 
 

@@ -192,8 +192,32 @@ extern "C" int mn_struct_layout(int which, size_t* offsets, int cap) {
       F(ldbeta) F(n_jobs) F(job) F(act_x) F(ld_act_x) F(act_pos) F(act_neg) F(act_y) F(ld_act_y) F(act_n) F(table) F(tok) F(vocab) F(top) F(idx)
 #undef F
   };
+  static const size_t streams[] = {
+#define F(f) MN_OFF(mn_streams_args, f)
+      F(src) F(src_row) F(src_stream) F(dst) F(S) F(n) F(mix) F(out) F(in) F(y) F(ldy) F(ye) F(ldye) F(slot_of) F(ew) F(top) F(one_plus) F(w)
+      F(eps) F(h) F(ldh) F(h16) F(ldh16)
+#undef F
+  };
+  static const size_t ms_layer[] = {
+#define F(f) MN_OFF(mn_ms_layer, f)
+      F(heads) F(kv_heads) F(dim) F(vdim) F(rot_dims) F(rot_interleaved) F(window) F(chunk) F(has_gate) F(v_mix) F(experts) F(top) F(expert_ff)
+      F(scale) F(rot_mag) F(v_lambda) F(rot_freq) F(sink) F(hc1_in) F(hc1_out) F(hc1_mix) F(hc2_in) F(hc2_out) F(hc2_mix) F(norm1) F(norm2)
+      F(w_in) F(b_in) F(q_norm) F(k_norm) F(w_o) F(w_router) F(w_gate_up) F(w_down)
+#undef F
+  };
+  static const size_t ms_model[] = {
+#define F(f) MN_OFF(mn_ms_model, f)
+      F(width) F(n_layers) F(streams) F(arith) F(norm_one_plus) F(eps) F(layers) F(final_w)
+#undef F
+  };
+  static const size_t ms_state[] = {
+#define F(f) MN_OFF(mn_ms_state, f)
+      F(k) F(v) F(n_seq) F(t_max)
+#undef F
+  };
   const size_t* tab[] = {skinny, rf, llm, semdec, comm, llm_tp, seq_layer, seq_model, seq_state, pmix_layer, pmix_model, pmix_state,
-                         hyb_layer, hyb_model, hyb_state, pn_layer, pn_model, pn_state, low_rank, rows_prep};
+                         hyb_layer, hyb_model, hyb_state, pn_layer, pn_model, pn_state, low_rank, rows_prep,
+                         streams, ms_layer, ms_model, ms_state};
   const int cnt[] = {(int)(sizeof(skinny) / sizeof(size_t)), (int)(sizeof(rf) / sizeof(size_t)), (int)(sizeof(llm) / sizeof(size_t)),
                      (int)(sizeof(semdec) / sizeof(size_t)), (int)(sizeof(comm) / sizeof(size_t)), (int)(sizeof(llm_tp) / sizeof(size_t)),
                      (int)(sizeof(seq_layer) / sizeof(size_t)), (int)(sizeof(seq_model) / sizeof(size_t)),
@@ -202,8 +226,10 @@ extern "C" int mn_struct_layout(int which, size_t* offsets, int cap) {
                      (int)(sizeof(hyb_layer) / sizeof(size_t)), (int)(sizeof(hyb_model) / sizeof(size_t)),
                      (int)(sizeof(hyb_state) / sizeof(size_t)), (int)(sizeof(pn_layer) / sizeof(size_t)),
                      (int)(sizeof(pn_model) / sizeof(size_t)), (int)(sizeof(pn_state) / sizeof(size_t)),
-                     (int)(sizeof(low_rank) / sizeof(size_t)), (int)(sizeof(rows_prep) / sizeof(size_t))};
-  MN_CHECK_ARG(which >= 0 && which < 20, "mn_struct_layout: unknown struct id");
+                     (int)(sizeof(low_rank) / sizeof(size_t)), (int)(sizeof(rows_prep) / sizeof(size_t)),
+                     (int)(sizeof(streams) / sizeof(size_t)), (int)(sizeof(ms_layer) / sizeof(size_t)),
+                     (int)(sizeof(ms_model) / sizeof(size_t)), (int)(sizeof(ms_state) / sizeof(size_t))};
+  MN_CHECK_ARG(which >= 0 && which < 24, "mn_struct_layout: unknown struct id");
   for (int i = 0; i < cnt[which] && i < cap; ++i) offsets[i] = tab[which][i];
   return cnt[which];
 }

@@ -730,7 +730,8 @@ int chan_rows(const ChanArgs& a, bool distinct, int n_runs, hipStream_t st) {
 template <bool VEC>
 __global__ __launch_bounds__(256) void gemv_glu_indexed_kernel(const float* __restrict__ A, int64_t lda, int a_div, const bf16_t* __restrict__ W,
                                                                int64_t ldw, int64_t w_bs, const int32_t* __restrict__ w_idx, int n_idx,
-                                                               float* __restrict__ C, int64_t ldc, int N, int K) {
+                                                               float* __restrict__ C, int64_t ldc, int N, int K,
+                                                               const float* __restrict__ x_scale) {
   const int z = blockIdx.y, n = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (n >= N || (unsigned)w_idx[z] >= (unsigned)n_idx) return;
   const float* ar = A + (int64_t)(z / a_div) * lda;
@@ -755,6 +756,7 @@ __global__ __launch_bounds__(256) void gemv_glu_indexed_kernel(const float* __re
   }
   sg = wave_sum(sg);
   su = wave_sum(su);
+  if (x_scale) { sg *= x_scale[z]; su *= x_scale[z]; }
   if (lane == 0) C[(int64_t)z * ldc + n] = silu_x(sg) * su;
 }
 
@@ -913,11 +915,16 @@ extern "C" int mn_channel_state_rows_scan(const float* qkv, int64_t ld, const fl
 
 extern "C" int mn_gemv_glu_indexed(const float* A, int64_t lda, int a_div, const uint16_t* W, int64_t ldw, int64_t w_bs, const int32_t* w_idx,
                                    int n_idx, float* C, int64_t ldc, int Z, int N, int K, void* stream) {
+  return mn_gemv_glu_indexed_scaled(A, lda, a_div, W, ldw, w_bs, w_idx, n_idx, nullptr, C, ldc, Z, N, K, stream);
+}
+
+extern "C" int mn_gemv_glu_indexed_scaled(const float* A, int64_t lda, int a_div, const uint16_t* W, int64_t ldw, int64_t w_bs, const int32_t* w_idx,
+                                          int n_idx, const float* x_scale, float* C, int64_t ldc, int Z, int N, int K, void* stream) {
   MN_CHECK_ARG(A && W && w_idx && C && a_div >= 1 && Z >= 1 && Z <= 65535 && N >= 1 && K >= 1 && n_idx >= 1, "mn_gemv_glu_indexed: bad args (Z=%d)", Z);
   const bool vec = (K % 8) == 0 && (ldw % 8) == 0 && (w_bs % 8) == 0 && (lda % 4) == 0 && (((uintptr_t)W | (uintptr_t)A) & 15) == 0;
   const dim3 grid((unsigned)mn_cdiv(N, 4), (unsigned)Z);
-  if (vec) hipLaunchKernelGGL((gemv_glu_indexed_kernel<true>), grid, dim3(256), 0, mn_stream(stream), A, lda, a_div, W, ldw, w_bs, w_idx, n_idx, C, ldc, N, K);
-  else hipLaunchKernelGGL((gemv_glu_indexed_kernel<false>), grid, dim3(256), 0, mn_stream(stream), A, lda, a_div, W, ldw, w_bs, w_idx, n_idx, C, ldc, N, K);
+  if (vec) hipLaunchKernelGGL((gemv_glu_indexed_kernel<true>), grid, dim3(256), 0, mn_stream(stream), A, lda, a_div, W, ldw, w_bs, w_idx, n_idx, C, ldc, N, K, x_scale);
+  else hipLaunchKernelGGL((gemv_glu_indexed_kernel<false>), grid, dim3(256), 0, mn_stream(stream), A, lda, a_div, W, ldw, w_bs, w_idx, n_idx, C, ldc, N, K, x_scale);
   MN_CHECK_LAUNCH("mn_gemv_glu_indexed");
   return MN_OK;
 }

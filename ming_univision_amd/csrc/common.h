@@ -180,8 +180,10 @@ typedef struct mn_g256 {
   // by a_scale[m] * w_scale[n] before bias / epilogue); no hi/lo rows, epilogues F32 (split-K allowed) and SWIGLU_BF16
   // grouped form: group g's weight scales at w_scale + g * w_sstride; a_scale is indexed by the SOURCE row (through a_rows when given)
   int f8; const float* a_scale; const float* w_scale; int64_t w_sstride;
+  const float* row_scale;                                // SWIGLU_BF16_SCALED: a factor per row POSITION, of the product's input (gate and up both take it)
 } mn_g256;
 enum { MN_G256_F32 = 0, MN_G256_BF16 = 1, MN_G256_BF16_GELU = 2, MN_G256_F32_RESID = 3, MN_G256_SWIGLU_SPLIT = 4,
-       MN_G256_F32_RESID_GATE = 5, MN_G256_SWIGLU_BF16 = 6, MN_G256_BF16_RELU2 = 7 };
+       MN_G256_F32_RESID_GATE = 5, MN_G256_SWIGLU_BF16 = 6, MN_G256_BF16_RELU2 = 7,
+       MN_G256_SWIGLU_BF16_SCALED = 8 };
 extern "C" int mn_gemm256_ex(const mn_g256* a, int epi, int ksplit, void* stream);
 extern "C" int mn_gemm256_slices(int K, int ksplit);

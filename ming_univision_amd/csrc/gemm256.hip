@@ -83,8 +83,8 @@ typedef mn_g256 G256;
 
 enum { E_F32 = MN_G256_F32, E_BF16 = MN_G256_BF16, E_BF16_GELU = MN_G256_BF16_GELU, E_F32_RESID = MN_G256_F32_RESID,
        E_SWIGLU_SPLIT = MN_G256_SWIGLU_SPLIT, E_F32_RESID_GATE = MN_G256_F32_RESID_GATE, E_SWIGLU_BF16 = MN_G256_SWIGLU_BF16,
-       E_BF16_RELU2 = MN_G256_BF16_RELU2 };
-__host__ __device__ constexpr bool epi_paired(int epi) { return epi == E_SWIGLU_SPLIT || epi == E_SWIGLU_BF16; }
+       E_BF16_RELU2 = MN_G256_BF16_RELU2, E_SWIGLU_BF16_SCALED = MN_G256_SWIGLU_BF16_SCALED };
+__host__ __device__ constexpr bool epi_paired(int epi) { return epi == E_SWIGLU_SPLIT || epi == E_SWIGLU_BF16 || epi == E_SWIGLU_BF16_SCALED; }
 
 __device__ __forceinline__ int lds_off(int buf, int op, int half) { return ((buf * 2 + op) * 2 + half) * HALF_BYTES; }
 
@@ -164,7 +164,11 @@ __device__ __forceinline__ void g256_emit(const G256& p, char* Cz, int m, int n,
       v = r * r;
     }
     *reinterpret_cast<u32x2*>(Cz + ((int64_t)m * p.ldc + n) * 2) = u32x2{cvt_pk_bf16(v.x, v.y), cvt_pk_bf16(v.z, v.w)};
-  } else if (EPI == E_SWIGLU_BF16) {   // y = silu(gate) * up as plain bf16 (the batched bf16 path)
+  } else if (EPI == E_SWIGLU_BF16 || EPI == E_SWIGLU_BF16_SCALED) {   // y = silu(gate) * up as plain bf16 (the batched bf16 path)
+    if (EPI == E_SWIGLU_BF16_SCALED) {                 // the input row's factor, applied to its products
+      const float rs = p.row_scale[m];
+      v *= rs; u *= rs;
+    }
     *reinterpret_cast<u32x2*>(Cz + ((int64_t)m * p.ldc + n) * 2) =
         u32x2{cvt_pk_bf16(silu_f(v.x) * u.x, silu_f(v.y) * u.y), cvt_pk_bf16(silu_f(v.z) * u.z, silu_f(v.w) * u.w)};
   } else {  // E_SWIGLU_SPLIT: y = silu(gate) * up, stored as bf16 hi rows and lo rows
@@ -452,6 +456,10 @@ static int g256_launch(const G256& a, int epi, int ksplit, hipStream_t st) {
     case E_F32_RESID_GATE: G256_GO(E_F32_RESID_GATE); break;
     case E_SWIGLU_BF16: G256_GO(E_SWIGLU_BF16); break;
     case E_BF16_RELU2: G256_GO(E_BF16_RELU2); break;
+    case E_SWIGLU_BF16_SCALED:
+      if (hilo || !a.row_scale) { mn_set_error("gemm256: the scaled SwiGLU epilogue takes plain rows and their factors"); return MN_EINVAL; }
+      hipLaunchKernelGGL((gemm256_kernel<E_SWIGLU_BF16_SCALED, false>), grid, dim3(512), 0, st, p);
+      break;
     default: mn_set_error("gemm256: bad epilogue %d", epi); return MN_EINVAL;
   }
 #undef G256_GO
@@ -608,6 +616,17 @@ extern "C" int mn_gemm256_grouped_tiles(const uint16_t* A, int64_t lda, int64_t 
                                         const uint16_t* W, int64_t ldw, int64_t w_gstride, const int32_t* off, const int32_t* cnt,
                                         int n_groups, const int32_t* tile_g, const int32_t* tile_m0, const int32_t* n_tiles,
                                         int max_mtiles, void* C, int64_t ldc, int64_t c_lo_off, int N, int K, int epi, void* stream) {
+  return mn_gemm256_grouped_tiles_scaled(A, lda, a_lo_off, a_rows_total, a_rows, W, ldw, w_gstride, off, cnt, n_groups, tile_g, tile_m0, n_tiles,
+                                         max_mtiles, nullptr, C, ldc, c_lo_off, N, K, epi, stream);
+}
+
+// The same with a factor per row position (epi 6 only: silu(s gate) * (s up) with s = row_scale[position])
+extern "C" int mn_gemm256_grouped_tiles_scaled(const uint16_t* A, int64_t lda, int64_t a_lo_off, int64_t a_rows_total, const int32_t* a_rows,
+                                               const uint16_t* W, int64_t ldw, int64_t w_gstride, const int32_t* off, const int32_t* cnt,
+                                               int n_groups, const int32_t* tile_g, const int32_t* tile_m0, const int32_t* n_tiles,
+                                               int max_mtiles, const float* row_scale, void* C, int64_t ldc, int64_t c_lo_off, int N, int K,
+                                               int epi, void* stream) {
+  MN_CHECK_ARG(!row_scale || (epi == E_SWIGLU_BF16 && a_lo_off == 0), "mn_gemm256_grouped_tiles_scaled: factors need epi 6 and plain bf16 rows");
   const bool paired = epi == E_SWIGLU_SPLIT || epi == E_SWIGLU_BF16;
   MN_CHECK_ARG(A && W && C && off && cnt && tile_g && tile_m0 && n_tiles && n_groups >= 1 && max_mtiles >= 1 && a_lo_off >= 0 &&
                    a_rows_total >= 1, "mn_gemm256_grouped_tiles: bad args");
@@ -623,7 +642,8 @@ extern "C" int mn_gemm256_grouped_tiles(const uint16_t* A, int64_t lda, int64_t 
   p.w_pair_rows = paired ? N : 0; p.M = (int)a_rows_total; p.N = N; p.K = K;
   p.g_off = off; p.g_cnt = cnt; p.w_gstride = w_gstride; p.a_rows = a_rows; p.n_groups = n_groups;
   p.tile_g = tile_g; p.tile_m0 = tile_m0; p.n_tiles = n_tiles; p.max_mtiles = max_mtiles;
-  const int rc = g256_launch(p, epi, 1, mn_stream(stream));
+  p.row_scale = row_scale;
+  const int rc = g256_launch(p, row_scale ? E_SWIGLU_BF16_SCALED : epi, 1, mn_stream(stream));
   if (rc < 0) return rc;
   MN_CHECK_LAUNCH("mn_gemm256_grouped_tiles");
   return MN_OK;

@@ -507,7 +507,13 @@ struct AttnTArgs {
   const float* sink;    // optional fp32 [H]: exp(sink[h]) joins the softmax's denominator of head h (no key, no value)
   float cap;            // > 0: every score s becomes cap * tanh(s / cap) before the softmax
   int64_t ldk, ldv;     // row strides of the key and value arenas (>= G * dim, G * vdim): a value arena may be a view into the key arena
+  int chunk;            // > 0: a position sees only its own chunk of `chunk` positions, counted from position 0 of the sequence
+  const float* gate; int64_t ldg;   // optional [M, H * vdim]: every result is multiplied by the sigmoid of its gate
 };
+
+__device__ __forceinline__ float gated(const AttnTArgs& a, float val, int row, int64_t col) {
+  return a.gate ? val * sigmoid_f(a.gate[(int64_t)row * a.ldg + col]) : val;
+}
 
 __device__ __forceinline__ float soft_cap(float s, float cap) { return cap > 0.f ? cap * tanhf(s / cap) : s; }
 
@@ -520,7 +526,12 @@ __device__ __forceinline__ float softmax_inv(float m, float l, const float* sink
   return f / (l * f + expf(sk - mm));
 }
 
+// the first position that position pos sees (of the tokens themselves); it never falls as pos grows
 __device__ __forceinline__ int win_t0(int pos, int window) { return window > 0 ? max(0, pos - window + 1) : 0; }
+__device__ __forceinline__ int first_key(const AttnTArgs& a, int pos) {
+  const int t = win_t0(pos, a.window);
+  return a.chunk > 0 ? max(t, pos - pos % a.chunk) : t;
+}
 __device__ __forceinline__ int win_nb(int pos, int window, int pool) {
   return (window > 0 && pool > 0 && pos - window + 1 >= 0) ? (pos - window + 1) / pool : 0;
 }
@@ -536,7 +547,7 @@ __global__ __launch_bounds__(256) void window_attn_tiled_kernel(AttnTArgs a) {
   const int nr = a.blk_tab ? min(a.blk_tab[2 * b + 1], a.rows_per_blk) : 1;
   const int nqv = nr * Rc;
   const int seq = a.row_seq[r0], pos0 = a.row_slot[r0], posL = pos0 + nr - 1;
-  const int nbL = win_nb(posL, a.window, a.pool), tF = win_t0(pos0, a.window);
+  const int nbL = win_nb(posL, a.window, a.pool), tF = first_key(a, pos0);
   const int nk = nbL + (posL - tF + 1);
   const int ntile = (nk + AKT - 1) / AKT, tps = (ntile + a.nsplit - 1) / a.nsplit;
   const int tile0 = sp * tps, tile1 = min(ntile, tile0 + tps);
@@ -611,7 +622,7 @@ __global__ __launch_bounds__(256) void window_attn_tiled_kernel(AttnTArgs a) {
         v += __shfl_xor(v, 2);
         if ((i & 3) == part) {
           const int pos = pos0 + i / Rc;
-          const bool see = valid && i < nqv && (j < nbL ? j < win_nb(pos, a.window, a.pool) : (t >= win_t0(pos, a.window) && t <= pos));
+          const bool see = valid && i < nqv && (j < nbL ? j < win_nb(pos, a.window, a.pool) : (t >= first_key(a, pos) && t <= pos));
           sc[i * AKT + key] = see ? soft_cap(v, a.cap) : -INFINITY;
         }
       }
@@ -686,9 +697,9 @@ __global__ __launch_bounds__(256) void window_attn_tiled_kernel(AttnTArgs a) {
       if (part_out) {
         part_out[2 * AQ + (int64_t)i * a.vdim + c0 + cc] = t;
       } else {
-        const float val = t * softmax_inv(st_m[i], st_l[i], a.sink, h0 + i % Rc) * a.out_scale;
         const int64_t col = (int64_t)(h0 + i % Rc) * a.vdim + c0 + cc;
         const int row = r0 + i / Rc;
+        const float val = gated(a, t * softmax_inv(st_m[i], st_l[i], a.sink, h0 + i % Rc) * a.out_scale, row, col);
         if (a.out) a.out[(int64_t)row * a.ldo + col] = val;
         if (a.out16) a.out16[(int64_t)row * a.ldo16 + col] = f32_to_bf16(val);
       }
@@ -720,7 +731,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(AttnTArgs a) {
   const int nr = a.blk_tab ? min(a.blk_tab[2 * b + 1], a.rows_per_blk) : 1;
   const int nqv = nr * Rc;
   const int seq = a.row_seq[r0], pos0 = a.row_slot[r0], posL = pos0 + nr - 1;
-  const int nbL = win_nb(posL, a.window, a.pool), tF = win_t0(pos0, a.window);
+  const int nbL = win_nb(posL, a.window, a.pool), tF = first_key(a, pos0);
   const int nk = nbL + (posL - tF + 1);
   const int ntile = (nk + KT - 1) / KT, tps = (ntile + a.nsplit - 1) / a.nsplit;
   const int t0 = sp * tps, t1 = min(ntile, t0 + tps);
@@ -748,7 +759,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(AttnTArgs a) {
     const int qv = 4 * g4 + i;
     mypos[i] = qv < nqv ? pos0 + qv / Rc : -1;              // -1: no such vector, it sees nothing
     my_nb[i] = qv < nqv ? win_nb(mypos[i], a.window, a.pool) : 0;
-    my_t0[i] = qv < nqv ? win_t0(mypos[i], a.window) : 0;
+    my_t0[i] = qv < nqv ? first_key(a, mypos[i]) : 0;
     mrun[i] = -INFINITY;
     lrun[i] = 0.f;
   }
@@ -834,7 +845,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(AttnTArgs a) {
       if (part_out) {
         part_out[2 * AQ + (int64_t)qv * a.vdim + d] = acc[c][i];
       } else {
-        const float val = acc[c][i] * inv;
+        const float val = gated(a, acc[c][i] * inv, row, col0 + d);
         if (a.out) a.out[(int64_t)row * a.ldo + col0 + d] = val;
         if (a.out16) a.out16[(int64_t)row * a.ldo16 + col0 + d] = f32_to_bf16(val);
       }
@@ -879,9 +890,9 @@ __global__ __launch_bounds__(256) void window_attn_merge_kernel(AttnTArgs a) {
     float t = 0.f;
 #pragma unroll 4
     for (int s = 0; s < a.nsplit; ++s) t = fmaf(src[s * stride], wgt[i * 64 + s], t);
-    const float val = t * softmax_inv(Ms[i], Ls[i], a.sink, h0 + i % Rc) * a.out_scale;
     const int64_t col = (int64_t)(h0 + i % Rc) * a.vdim + c;
     const int row = r0 + i / Rc;
+    const float val = gated(a, t * softmax_inv(Ms[i], Ls[i], a.sink, h0 + i % Rc) * a.out_scale, row, col);
     if (a.out) a.out[(int64_t)row * a.ldo + col] = val;
     if (a.out16) a.out16[(int64_t)row * a.ldo16 + col] = f32_to_bf16(val);
   }
@@ -983,8 +994,10 @@ __global__ __launch_bounds__(256) void mingru_pass3_kernel(MinGruArgs a) {
   }
 }
 
-// one wave per row: `top` rounds of arg-max (ties: the lower index), then the softmax over the chosen logits.  Lane l owns the
+// one wave per row: `top` rounds of arg-max (ties: the lower index), then the softmax over the chosen logits (SIGMOID: every chosen
+// logit's sigmoid as it is).  Lane l owns the
 // logits l, l + 64, ... and a bit per owned logit that says it has been chosen (E <= 4096).
+template <bool SIGMOID>
 __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restrict__ logits, int64_t ld, int M, int E, int top,
                                                           int32_t* __restrict__ idx, float* __restrict__ w, const float* __restrict__ sx,
                                                           int64_t ldsx, float* __restrict__ sy, int64_t ldsy, int sn) {
@@ -1015,20 +1028,22 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restric
     }
     if ((bi & 63) == lane) taken |= (uint64_t)1 << (bi >> 6);
     if (k == 0) first = best;
-    const float p = expf(best - first);
+    const float p = SIGMOID ? sigmoid_f(best) : expf(best - first);
     sum += p;
     if (lane == 0) { ir[k] = bi; wr[k] = p; }
   }
+  if (SIGMOID) return;
   // lane 0 wrote the unnormalised weights and is the one that scales them
   if (lane == 0)
     for (int k = 0; k < top; ++k) wr[k] = wr[k] / sum;
 }
 
-__global__ __launch_bounds__(256) void silu_mul_kernel(const float* __restrict__ x, int64_t ldx, float* __restrict__ y, int64_t ldy,
-                                                       bf16_t* __restrict__ y16, int64_t ldy16, int n) {
+__global__ __launch_bounds__(256) void silu_mul_kernel(const float* __restrict__ x, int64_t ldx, const float* __restrict__ s,
+                                                       float* __restrict__ y, int64_t ldy, bf16_t* __restrict__ y16, int64_t ldy16, int n) {
   const int m = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
   if (c >= n) return;
-  const float o = silu_f(x[(int64_t)m * ldx + c]) * x[(int64_t)m * ldx + n + c];
+  const float f = s ? s[m] : 1.0f;
+  const float o = silu_f(f * x[(int64_t)m * ldx + c]) * (f * x[(int64_t)m * ldx + n + c]);
   if (y) y[(int64_t)m * ldy + c] = o;
   if (y16) y16[(int64_t)m * ldy16 + c] = f32_to_bf16(o);
 }
@@ -1262,6 +1277,17 @@ extern "C" int mn_window_pool_attn_blocks_cap(const float* q, int64_t ldq, const
                                               int vdim, int t_max, int n_pool_max, int window, int pool, float out_scale, float* out, int64_t ldo,
                                               uint16_t* out16, int64_t ldo16, int nsplit, void* workspace, size_t workspace_bytes, int variant,
                                               void* stream) {
+  return mn_window_pool_attn_blocks_gate(q, ldq, k_arena, ldk, v_arena, ldv, pk, pv, sink, softcap, 0, nullptr, 0, row_seq, row_slot, blk_tab, n_blk,
+                                         one_row, H, G, dim, vdim, t_max, n_pool_max, window, pool, out_scale, out, ldo, out16, ldo16, nsplit,
+                                         workspace, workspace_bytes, variant, stream);
+}
+
+extern "C" int mn_window_pool_attn_blocks_gate(const float* q, int64_t ldq, const float* k_arena, int64_t ldk, const float* v_arena, int64_t ldv,
+                                               const float* pk, const float* pv, const float* sink, float softcap, int chunk, const float* gate,
+                                               int64_t ldgate, const int32_t* row_seq, const int32_t* row_slot, const int32_t* blk_tab, int n_blk,
+                                               int one_row, int H, int G, int dim, int vdim, int t_max, int n_pool_max, int window, int pool,
+                                               float out_scale, float* out, int64_t ldo, uint16_t* out16, int64_t ldo16, int nsplit, void* workspace,
+                                               size_t workspace_bytes, int variant, void* stream) {
   if (ldk <= 0) ldk = (int64_t)G * dim;
   if (ldv <= 0) ldv = (int64_t)G * vdim;
   MN_CHECK_ARG(ldk >= (int64_t)G * dim && ldv >= (int64_t)G * vdim && ((dim % 4) != 0 || (ldk % 4) == 0) && ((vdim % 4) != 0 || (ldv % 4) == 0) &&
@@ -1273,12 +1299,15 @@ extern "C" int mn_window_pool_attn_blocks_cap(const float* q, int64_t ldq, const
                "mn_window_pool_attn_blocks: bad args (vdim=%d: at most 512; nsplit=%d: at most 64)", vdim, nsplit);
   MN_CHECK_ARG(pool == 0 || (window > 0 && pk && pv && n_pool_max >= 1), "mn_window_pool_attn_blocks: pooled blocks need a window and their arenas");
   MN_CHECK_ARG(one_row || blk_tab, "mn_window_pool_attn_blocks: runs of several rows need their table");
+  MN_CHECK_ARG(chunk >= 0 && (chunk == 0 || pool == 0) && (!gate || ldgate >= (int64_t)H * vdim),
+               "mn_window_pool_attn_blocks: chunks go without pooled blocks; a gate row holds H * vdim values");
   const AttnShape sh = attn_shape(H, G, one_row);
   MN_CHECK_ARG((int64_t)G * sh.chunks <= 65535, "mn_window_pool_attn_blocks: too many heads");
   MN_CHECK_ARG(nsplit == 1 || (workspace && workspace_bytes >= mn_window_attn_workspace_bytes(n_blk, H, G, vdim, one_row, nsplit)),
                "mn_window_pool_attn_blocks: workspace too small");
   AttnTArgs a{q, ldq, k_arena, v_arena, pool ? pk : nullptr, pool ? pv : nullptr, row_seq, row_slot, one_row ? nullptr : blk_tab, H, G, dim, vdim,
-              t_max, n_pool_max, window, pool, sh.rows, sh.hpc, nsplit, out_scale, out, ldo, out16, ldo16, (float*)workspace, sink, softcap, ldk, ldv};
+              t_max, n_pool_max, window, pool, sh.rows, sh.hpc, nsplit, out_scale, out, ldo, out16, ldo16, (float*)workspace, sink, softcap, ldk, ldv,
+              chunk, gate, ldgate};
   // values that are a view of the keys (one key/value head, the same arena and stride): the matrix-core kernel stages one tile for both
   const bool vk = G == 1 && k_arena == v_arena && ldk == ldv && vdim <= dim && !pool;
   const bool mfma_fits = vk ? (dim <= 640 && sh.aq == 16) : (!one_row && dim <= 256 && vdim <= 256);
@@ -1375,9 +1404,17 @@ extern "C" int mn_mingru_rows_scan(const float* zx, int64_t ldzx, const float* g
 
 extern "C" int mn_router_topk_rows(const float* logits, int64_t ld, int M, int E, int top, int32_t* idx, float* w, void* stream) {
   MN_CHECK_ARG(logits && idx && w && M >= 1 && E >= 1 && E <= 4096 && top >= 1 && top <= E, "mn_router_topk_rows: bad args (E=%d top=%d)", E, top);
-  hipLaunchKernelGGL(router_topk_kernel, dim3((unsigned)mn_cdiv(M, 4)), dim3(256), 0, mn_stream(stream), logits, ld, M, E, top, idx, w,
+  hipLaunchKernelGGL((router_topk_kernel<false>), dim3((unsigned)mn_cdiv(M, 4)), dim3(256), 0, mn_stream(stream), logits, ld, M, E, top, idx, w,
                      (const float*)nullptr, (int64_t)0, (float*)nullptr, (int64_t)0, 0);
   MN_CHECK_LAUNCH("mn_router_topk_rows");
+  return MN_OK;
+}
+
+extern "C" int mn_router_sigmoid_topk_rows(const float* logits, int64_t ld, int M, int E, int top, int32_t* idx, float* w, void* stream) {
+  MN_CHECK_ARG(logits && idx && w && M >= 1 && E >= 1 && E <= 4096 && top >= 1 && top <= E, "mn_router_sigmoid_topk_rows: bad args (E=%d top=%d)", E, top);
+  hipLaunchKernelGGL((router_topk_kernel<true>), dim3((unsigned)mn_cdiv(M, 4)), dim3(256), 0, mn_stream(stream), logits, ld, M, E, top, idx, w,
+                     (const float*)nullptr, (int64_t)0, (float*)nullptr, (int64_t)0, 0);
+  MN_CHECK_LAUNCH("mn_router_sigmoid_topk_rows");
   return MN_OK;
 }
 
@@ -1385,7 +1422,7 @@ extern "C" int mn_router_topk_silu_rows(const float* logits, int64_t ld, int M, 
                                         int64_t ldx, float* y, int64_t ldy, int n, void* stream) {
   MN_CHECK_ARG(logits && idx && w && x && y && M >= 1 && E >= 1 && E <= 4096 && top >= 1 && top <= E && n >= 1 &&
                    mn_cdiv(M, 4) + (int64_t)M * mn_cdiv(n, 256) <= 0x7fffffff, "mn_router_topk_silu_rows: bad args (E=%d top=%d)", E, top);
-  hipLaunchKernelGGL(router_topk_kernel, dim3((unsigned)(mn_cdiv(M, 4) + (int64_t)M * mn_cdiv(n, 256))), dim3(256), 0, mn_stream(stream), logits,
+  hipLaunchKernelGGL((router_topk_kernel<false>), dim3((unsigned)(mn_cdiv(M, 4) + (int64_t)M * mn_cdiv(n, 256))), dim3(256), 0, mn_stream(stream), logits,
                      ld, M, E, top, idx, w, x, ldx, y, ldy, n);
   MN_CHECK_LAUNCH("mn_router_topk_silu_rows");
   return MN_OK;
@@ -1393,9 +1430,14 @@ extern "C" int mn_router_topk_silu_rows(const float* logits, int64_t ld, int M, 
 
 extern "C" int mn_silu_mul_rows(const float* x, int64_t ldx, float* y, int64_t ldy, uint16_t* y16, int64_t ldy16, int M, int n,
                                 void* stream) {
+  return mn_silu_mul_rows_scaled(x, ldx, nullptr, y, ldy, y16, ldy16, M, n, stream);
+}
+
+extern "C" int mn_silu_mul_rows_scaled(const float* x, int64_t ldx, const float* x_scale, float* y, int64_t ldy, uint16_t* y16, int64_t ldy16,
+                                       int M, int n, void* stream) {
   MN_CHECK_ARG(x && (y || y16) && M >= 1 && M <= 65535 && n >= 1, "mn_silu_mul_rows: bad args");
-  hipLaunchKernelGGL(silu_mul_kernel, dim3((unsigned)mn_cdiv(n, 256), (unsigned)M), dim3(256), 0, mn_stream(stream), x, ldx, y, ldy, y16,
-                     ldy16, n);
+  hipLaunchKernelGGL(silu_mul_kernel, dim3((unsigned)mn_cdiv(n, 256), (unsigned)M), dim3(256), 0, mn_stream(stream), x, ldx, x_scale, y, ldy,
+                     y16, ldy16, n);
   MN_CHECK_LAUNCH("mn_silu_mul_rows");
   return MN_OK;
 }

@@ -115,44 +115,94 @@ struct ProjNormArgs {
   int H, G, dim, vdim, rot_dims, interleaved, t_max;
   const bf16_t *q_norm, *k_norm;
   const float* freq;
-  float eps, q_scale;
+  float mag, eps, q_scale;
   const int32_t *row_seq, *row_slot;
   float* q_out; int64_t ldq;
   float* k_arena; int64_t ldk;
   float* v_arena; int64_t ldv;
+  float* v_keep; int64_t ldvk;               // optional: the row's values as projected, for layers that mix them in
+  const float* v_first; int64_t ldvf;        // optional: values to mix in, v <- (1 - v_lambda) v + v_lambda v_first
+  float v_lambda;
 };
 
-__global__ __launch_bounds__(256) void proj_norm_rope_append_kernel(ProjNormArgs a) {
-  __shared__ float red[4];
-  const int m = blockIdx.x, tid = threadIdx.x;
+// One workgroup per row.  The row's cosines and sines (of one head's pairs: every head turns alike) are computed once into LDS
+// [2 rot_dims / 2].  GW = 4: groups of four consecutive values, a group of the first half of a head's pairs writes its partners too.
+template <int NT, int GW>
+__global__ __launch_bounds__(NT) void proj_norm_rope_append_kernel(ProjNormArgs a) {
+  extern __shared__ __align__(16) float cs[];
+  __shared__ float red[NT / 64];
+  typedef float vec_t __attribute__((ext_vector_type(4)));
+  const int m = blockIdx.x, tid = threadIdx.x, half = a.rot_dims >> 1;
   const int nq = a.H * a.dim, nk = a.G * a.dim, nv = a.G * a.vdim;
   const float* row = a.qkv + (int64_t)m * a.ld;
   const int seq = a.row_seq[m], pos = a.row_slot[m];
+  for (int i = tid; i < half; i += NT) {
+    const float ang = (float)pos * a.freq[i];
+    cs[i] = cosf(ang) * a.mag;
+    cs[half + i] = sinf(ang) * a.mag;
+  }
+  auto square_sum = [&](const float* p, int n) {
+    float ss = 0.f;
+    if constexpr (GW == 4) {
+      for (int e = 4 * tid; e < n; e += 4 * NT) {
+        const vec_t v = *reinterpret_cast<const vec_t*>(p + e);
+        ss = fmaf(v.x, v.x, ss); ss = fmaf(v.y, v.y, ss); ss = fmaf(v.z, v.z, ss); ss = fmaf(v.w, v.w, ss);
+      }
+    } else {
+      for (int e = tid; e < n; e += NT) ss = fmaf(p[e], p[e], ss);
+    }
+    return ss;
+  };
   float rq = 1.0f, rk = 1.0f;
-  if (a.q_norm) {
-    float ss = 0.f;
-    for (int e = tid; e < nq; e += 256) ss = fmaf(row[e], row[e], ss);
-    rq = 1.0f / sqrtf(block_sum(ss, red) / (float)nq + a.eps);
-  }
-  if (a.k_norm) {
-    float ss = 0.f;
-    for (int e = tid; e < nk; e += 256) ss = fmaf(row[nq + e], row[nq + e], ss);
-    rk = 1.0f / sqrtf(block_sum(ss, red) / (float)nk + a.eps);
-  }
-  for (int e = tid; e < nq; e += 256) {
-    const int d = e % a.dim, e0 = e - d;
-    auto at = [&](int j) { return row[e0 + j] * rq * (a.q_norm ? bf16_to_f32(a.q_norm[e0 + j]) : 1.0f); };
-    const float v = d < a.rot_dims ? rotate_value(at, d, a.rot_dims, a.interleaved, a.freq, pos) : at(d);
-    a.q_out[(int64_t)m * a.ldq + e] = v * a.q_scale;
-  }
+  if (a.q_norm) rq = 1.0f / sqrtf(block_sum(square_sum(row, nq), red) / (float)nq + a.eps);
+  if (a.k_norm) rk = 1.0f / sqrtf(block_sum(square_sum(row + nq, nk), red) / (float)nk + a.eps);
+  __syncthreads();
   float* kd = a.k_arena + ((int64_t)seq * a.t_max + pos) * a.ldk;
-  for (int e = tid; e < nk; e += 256) {
-    const int d = e % a.dim, e0 = e - d;
-    auto at = [&](int j) { return row[nq + e0 + j] * rk * (a.k_norm ? bf16_to_f32(a.k_norm[e0 + j]) : 1.0f); };
-    kd[e] = d < a.rot_dims ? rotate_value(at, d, a.rot_dims, a.interleaved, a.freq, pos) : at(d);
-  }
+  // one projection: n values at src with their norm weights (w NULL: none) to dst, times scale
+  auto turn = [&](const float* src, int n, const bf16_t* w, float r, float scale, float* dst) {
+    if constexpr (GW == 4) {
+      auto load = [&](int e) {
+        vec_t v = *reinterpret_cast<const vec_t*>(src + e) * r;
+        if (w) {
+          const uint2 u = *reinterpret_cast<const uint2*>(w + e);
+          v *= vec_t{bf16lo_to_f32(u.x), bf16hi_to_f32(u.x), bf16lo_to_f32(u.y), bf16hi_to_f32(u.y)};
+        }
+        return v;
+      };
+      for (int e = 4 * tid; e < n; e += 4 * NT) {
+        const int d = e % a.dim;
+        if (d >= a.rot_dims) {
+          *reinterpret_cast<vec_t*>(dst + e) = load(e) * scale;
+        } else if (d < half) {
+          const vec_t u = load(e), v = load(e + half), c = *reinterpret_cast<const vec_t*>(cs + d), s = *reinterpret_cast<const vec_t*>(cs + half + d);
+          *reinterpret_cast<vec_t*>(dst + e) = (u * c - v * s) * scale;
+          *reinterpret_cast<vec_t*>(dst + e + half) = (v * c + u * s) * scale;
+        }
+      }
+    } else {
+      for (int e = tid; e < n; e += NT) {
+        const int d = e % a.dim, e0 = e - d;
+        auto at = [&](int j) { return src[e0 + j] * r * (w ? bf16_to_f32(w[e0 + j]) : 1.0f); };
+        float v = at(d);
+        if (d < a.rot_dims) {
+          const bool first = a.interleaved ? (d & 1) == 0 : d < half;
+          const int i = a.interleaved ? (d >> 1) : (first ? d : d - half);
+          const float p = at(a.interleaved ? (d ^ 1) : (first ? d + half : d - half));
+          v = first ? v * cs[i] - p * cs[half + i] : v * cs[i] + p * cs[half + i];
+        }
+        dst[e] = v * scale;
+      }
+    }
+  };
+  turn(row, nq, a.q_norm, rq, a.q_scale, a.q_out + (int64_t)m * a.ldq);
+  turn(row + nq, nk, a.k_norm, rk, 1.0f, kd);
   float* vd = a.v_arena + ((int64_t)seq * a.t_max + pos) * a.ldv;
-  for (int e = tid; e < nv; e += 256) vd[e] = row[nq + nk + e];
+  for (int e = tid; e < nv; e += NT) {
+    float v = row[nq + nk + e];
+    if (a.v_keep) a.v_keep[(int64_t)m * a.ldvk + e] = v;
+    if (a.v_first) v = (1.0f - a.v_lambda) * v + a.v_lambda * a.v_first[(int64_t)m * a.ldvf + e];
+    vd[e] = v;
+  }
 }
 
 struct LatentRopeArgs {
@@ -551,13 +601,33 @@ extern "C" int mn_proj_norm_rope_append(const float* qkv, int64_t ldqkv, int M, 
                                         const uint16_t* k_norm, float eps, int rot_dims, int interleaved, const float* freq, float q_scale,
                                         const int32_t* row_seq, const int32_t* row_slot, float* q_out, int64_t ldq, float* k_arena,
                                         int64_t ldk, float* v_arena, int64_t ldv, int t_max, void* stream) {
+  return mn_proj_norm_rope_mix_append(qkv, ldqkv, M, H, G, dim, vdim, q_norm, k_norm, eps, rot_dims, interleaved, freq, 1.0f, q_scale, nullptr, 0,
+                                      nullptr, 0, 0.0f, row_seq, row_slot, q_out, ldq, k_arena, ldk, v_arena, ldv, t_max, stream);
+}
+
+extern "C" int mn_proj_norm_rope_mix_append(const float* qkv, int64_t ldqkv, int M, int H, int G, int dim, int vdim, const uint16_t* q_norm,
+                                            const uint16_t* k_norm, float eps, int rot_dims, int interleaved, const float* freq, float rot_mag,
+                                            float q_scale, float* v_keep, int64_t ldvk, const float* v_first, int64_t ldvf, float v_lambda,
+                                            const int32_t* row_seq, const int32_t* row_slot, float* q_out, int64_t ldq, float* k_arena,
+                                            int64_t ldk, float* v_arena, int64_t ldv, int t_max, void* stream) {
   MN_CHECK_ARG(qkv && row_seq && row_slot && q_out && k_arena && v_arena && M >= 1 && H >= 1 && G >= 1 && dim >= 1 && vdim >= 1 && t_max >= 1 &&
-                   rot_dims >= 0 && rot_dims <= dim && (rot_dims % 2) == 0 && (rot_dims == 0 || freq) && ldk >= (int64_t)G * dim &&
-                   ldv >= (int64_t)G * vdim,
+                   rot_dims >= 0 && rot_dims <= dim && rot_dims <= 8192 && (rot_dims % 2) == 0 && (rot_dims == 0 || freq) && ldk >= (int64_t)G * dim &&
+                   ldv >= (int64_t)G * vdim && (!v_keep || ldvk >= (int64_t)G * vdim) && (!v_first || ldvf >= (int64_t)G * vdim),
                "mn_proj_norm_rope_append: bad args (rot_dims=%d of dim=%d)", rot_dims, dim);
-  ProjNormArgs a{qkv, ldqkv, H, G, dim, vdim, rot_dims, interleaved ? 1 : 0, t_max, q_norm, k_norm, freq, eps, q_scale, row_seq, row_slot,
-                 q_out, ldq, k_arena, ldk, v_arena, ldv};
-  hipLaunchKernelGGL(proj_norm_rope_append_kernel, dim3((unsigned)M), dim3(256), 0, mn_stream(stream), a);
+  ProjNormArgs a{qkv, ldqkv, H, G, dim, vdim, rot_dims, interleaved ? 1 : 0, t_max, q_norm, k_norm, freq, rot_mag, eps, q_scale, row_seq, row_slot,
+                 q_out, ldq, k_arena, ldk, v_arena, ldv, v_keep, ldvk, v_first, ldvf, v_lambda};
+  const bool vec = !interleaved && (dim % 4) == 0 && (rot_dims % 8) == 0 && (ldqkv % 4) == 0 && (ldq % 4) == 0 && (ldk % 4) == 0 &&
+                   (((uintptr_t)qkv | (uintptr_t)q_out | (uintptr_t)k_arena) & 15) == 0 && (((uintptr_t)q_norm | (uintptr_t)k_norm) & 7) == 0;
+  const size_t lds = (size_t)rot_dims * sizeof(float);
+  hipStream_t st = mn_stream(stream);
+  // few rows: the row's latency is the launch, so a row gets 16 waves
+  if (M <= 64) {
+    if (vec) hipLaunchKernelGGL((proj_norm_rope_append_kernel<1024, 4>), dim3((unsigned)M), dim3(1024), lds, st, a);
+    else hipLaunchKernelGGL((proj_norm_rope_append_kernel<1024, 1>), dim3((unsigned)M), dim3(1024), lds, st, a);
+  } else {
+    if (vec) hipLaunchKernelGGL((proj_norm_rope_append_kernel<256, 4>), dim3((unsigned)M), dim3(256), lds, st, a);
+    else hipLaunchKernelGGL((proj_norm_rope_append_kernel<256, 1>), dim3((unsigned)M), dim3(256), lds, st, a);
+  }
   MN_CHECK_LAUNCH("mn_proj_norm_rope_append");
   return MN_OK;
 }

@@ -311,7 +311,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int32_t* __restric
                                                         int32_t* __restrict__ perm, int32_t* __restrict__ slot_of,
                                                         int n_slot, int tile_rows, int32_t* __restrict__ tile_g,
                                                         int32_t* __restrict__ tile_m0, int32_t* __restrict__ n_tiles,
-                                                        int g_lo, int g_hi) {
+                                                        int g_lo, int g_hi, const float* __restrict__ w,
+                                                        float* __restrict__ w_sorted) {
   __shared__ int cnt[128], off[129], cur[128], toff[129], wtot[2];
   const int tid = threadIdx.x, lane = tid & 63;
   if (tid < 128) { cnt[tid] = 0; cur[tid] = 0; }
@@ -354,6 +355,7 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int32_t* __restric
     const int pos = off[e] + atomicAdd(&cur[e], 1);
     perm[pos] = i / n_slot;       // sorted position -> token
     slot_of[i] = pos;             // (token, pick) -> sorted position
+    if (w_sorted) w_sorted[pos] = w[i];
   }
 }
 
@@ -362,7 +364,7 @@ extern "C" int mn_moe_sort(const int32_t* topk_idx, int T, int n_slot, int n_gro
   MN_CHECK_ARG(topk_idx && counts && offsets && perm && slot_of && T >= 1 && n_slot >= 1 && n_groups >= 1 && n_groups <= 128 &&
                    (int64_t)T * n_slot <= 65536, "mn_moe_sort: bad args");
   hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, mn_stream(stream), topk_idx, T * n_slot, n_groups, counts,
-                     offsets, perm, slot_of, n_slot, 0, (int32_t*)nullptr, (int32_t*)nullptr, (int32_t*)nullptr, 0, 0);
+                     offsets, perm, slot_of, n_slot, 0, (int32_t*)nullptr, (int32_t*)nullptr, (int32_t*)nullptr, 0, 0, (const float*)nullptr, (float*)nullptr);
   MN_CHECK_LAUNCH("mn_moe_sort");
   return MN_OK;
 }
@@ -375,8 +377,21 @@ extern "C" int mn_moe_sort_tiles(const int32_t* topk_idx, int T, int n_slot, int
   MN_CHECK_ARG(topk_idx && counts && offsets && perm && slot_of && tile_g && tile_m0 && n_tiles && tile_rows >= 1 && T >= 1 &&
                    n_slot >= 1 && n_groups >= 1 && n_groups <= 128 && (int64_t)T * n_slot <= 65536, "mn_moe_sort_tiles: bad args");
   hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, mn_stream(stream), topk_idx, T * n_slot, n_groups, counts,
-                     offsets, perm, slot_of, n_slot, tile_rows, tile_g, tile_m0, n_tiles, 0, n_groups);
+                     offsets, perm, slot_of, n_slot, tile_rows, tile_g, tile_m0, n_tiles, 0, n_groups, (const float*)nullptr, (float*)nullptr);
   MN_CHECK_LAUNCH("mn_moe_sort_tiles");
+  return MN_OK;
+}
+
+// mn_moe_sort (tile_g NULL) or mn_moe_sort_tiles that also brings the picks' weights into the sorted order
+extern "C" int mn_moe_sort_weights(const int32_t* topk_idx, const float* topk_w, int T, int n_slot, int n_groups, int32_t* counts,
+                                   int32_t* offsets, int32_t* perm, int32_t* slot_of, float* w_sorted, int tile_rows, int32_t* tile_g,
+                                   int32_t* tile_m0, int32_t* n_tiles, void* stream) {
+  MN_CHECK_ARG(topk_idx && topk_w && counts && offsets && perm && slot_of && w_sorted && T >= 1 && n_slot >= 1 && n_groups >= 1 &&
+                   n_groups <= 128 && (int64_t)T * n_slot <= 65536 && (!tile_g || (tile_m0 && n_tiles && tile_rows >= 1)),
+               "mn_moe_sort_weights: bad args");
+  hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, mn_stream(stream), topk_idx, T * n_slot, n_groups, counts, offsets, perm,
+                     slot_of, n_slot, tile_rows, tile_g, tile_m0, n_tiles, 0, n_groups, topk_w, w_sorted);
+  MN_CHECK_LAUNCH("mn_moe_sort_weights");
   return MN_OK;
 }
 
@@ -390,7 +405,7 @@ extern "C" int mn_ep_dispatch(const int32_t* topk_idx, int T, int n_slot, int n_
                    n_slot >= 1 && n_experts >= 1 && n_experts <= 128 && (int64_t)T * n_slot <= 65536 && expert0 >= 0 && n_local >= 1 &&
                    expert0 + n_local <= n_experts, "mn_ep_dispatch: bad args");
   hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, mn_stream(stream), topk_idx, T * n_slot, n_experts, counts,
-                     offsets, perm, slot_of, n_slot, tile_rows, tile_g, tile_m0, n_tiles, expert0, expert0 + n_local);
+                     offsets, perm, slot_of, n_slot, tile_rows, tile_g, tile_m0, n_tiles, expert0, expert0 + n_local, (const float*)nullptr, (float*)nullptr);
   MN_CHECK_LAUNCH("mn_ep_dispatch");
   return MN_OK;
 }

@@ -44,7 +44,7 @@ def load_safetensors_dir(path):
 def load_model(path, dtype="bf16", device="cuda", **kw):
     """The served model of a checkpoint directory, its class chosen by config.json (configuration.MODEL_REGISTRY):
     "pizitar" -> PizitarForCausalLM, "sakinex" -> SakinexForCausalLM, "zuzenex" -> ZuzenexForCausalLM, "daberax" -> DaberaxForCausalLM,
-    "sabezen" -> SabezenForCausalLM (dtype "bf16" | "f32" = the matrix-product arithmetic; kw: t_max,
+    "sabezen" -> SabezenForCausalLM, "fegarax" -> FegaraxForCausalLM (dtype "bf16" | "f32" = the matrix-product arithmetic; kw: t_max,
     eos_token_id),
     "ming_univision" -> MingUniVisionInfer (dtype = the weight format)."""
     from .configuration import config_from_pretrained
@@ -64,6 +64,9 @@ def load_model(path, dtype="bf16", device="cuda", **kw):
     if name == "sabezen":
         from .sabezen import SabezenForCausalLM
         return SabezenForCausalLM.from_pretrained(path, device=device, arith=dtype, **kw)
+    if name == "fegarax":
+        from .fegarax import FegaraxForCausalLM
+        return FegaraxForCausalLM.from_pretrained(path, device=device, arith=dtype, **kw)
     return MingUniVisionInfer(path, dtype=dtype, device=device, **kw)
 
 

@@ -146,14 +146,6 @@ class SabezenDecoder(HybridSteps, SeqDecoder):
         self._ws, self._decode_tabs = {}, {}
         self._init_state()
 
-    # ---- caches and states ---------------------------------------------------------------------------------------------------
-    PER_TOKEN = ("k", "v")                              # arenas with one row per cached token
-
-    def _state_shapes(self, n_seq):
-        """Per layer: {name: shape or None}."""
-        return [{k: (None if d.get(k) is None else ((n_seq, self.t_max) if k in self.PER_TOKEN else (n_seq,)) + tuple(d[k]))
-                 for k in self.STATE_KEYS} for d in self.dims]
-
     # ---- construction ---------------------------------------------------------------------------------------------------------
     @classmethod
     def from_pretrained(cls, path, device="cuda", **kw):

@@ -174,14 +174,16 @@ class SequenceArenas:
         self._bind_state()
 
 
-class HybridSteps(SequenceArenas):
-    """A decoder whose passes run on the hybrid-mixer step function (mn_hyb_step): `struct` = its HybModel, `runs` = the layer of every
-    layer run, `chunk_rows` where the recurrences take chunk tables."""
-    STATE_KEYS = ("k", "v", "lin", "conv")
-    STATE_STRUCT = _lib.HybState
+class NativeSteps(SequenceArenas):
+    """A decoder whose passes run on one of the library's step functions: the checks of a pass's arguments and the buffers it needs.  The
+    step function's class gives `_workspace_bytes` and `_launch` (the call itself)."""
 
-    def _workspace_bytes(self, rows, max_len):
-        return lib().mn_hyb_workspace_bytes(C.byref(self.struct), rows)
+    PER_TOKEN = ("k", "v")                              # arenas with one row per cached token
+
+    def _state_shapes(self, n_seq):
+        """Per layer: {name: shape or None} of `dims` = per layer {state key: shape behind the sequence axis (per token for PER_TOKEN)}."""
+        return [{k: (None if d.get(k) is None else ((n_seq, self.t_max) if k in self.PER_TOKEN else (n_seq,)) + tuple(d[k]))
+                 for k in self.STATE_KEYS} for d in self.dims]
 
     def max_rows(self):
         """Rows of one pass: the (row, expert) pairs of a pass are at most 65535."""
@@ -214,12 +216,37 @@ class HybridSteps(SequenceArenas):
             assert trace.dtype == torch.float32 and trace.is_contiguous() and tuple(trace.shape) == (self.n_trace, M, self.cfg.width)
         if ws is None:
             ws = self._workspace(M, max_len)
-        use_chunks = chunk_tab is not None and not distinct
-        check(lib().mn_hyb_step(C.byref(self.struct), C.byref(self.state), ptr(x), x.stride(0), M, ptr(row_tok), ptr(row_seq), ptr(row_slot),
-                                ptr(row_back), None if distinct else ptr(blk_tab), M if distinct else blk_tab.shape[0],
-                                ptr(chunk_tab) if use_chunks else None, chunk_tab.shape[0] if use_chunks else 0, max_len,
-                                1 if distinct else 0, ptr(out), ptr(trace), ptr(ws), ws.numel(), current_stream()), "mn_hyb_step")
+        self._launch(x, row_tok, row_seq, row_slot, row_back, None if distinct else blk_tab, M if distinct else blk_tab.shape[0],
+                     None if distinct else chunk_tab, max_len, 1 if distinct else 0, out, trace, ws)
         return out
+
+
+class HybridSteps(NativeSteps):
+    """Passes on the hybrid-mixer step function (mn_hyb_step): `struct` = the decoder's HybModel, `runs` = the layer of every layer run,
+    `chunk_rows` where the recurrences take chunk tables."""
+    STATE_KEYS = ("k", "v", "lin", "conv")
+    STATE_STRUCT = _lib.HybState
+
+    def _workspace_bytes(self, rows, max_len):
+        return lib().mn_hyb_workspace_bytes(C.byref(self.struct), rows)
+
+    def _launch(self, x, row_tok, row_seq, row_slot, row_back, blk_tab, n_blk, chunk_tab, max_len, flags, out, trace, ws):
+        check(lib().mn_hyb_step(C.byref(self.struct), C.byref(self.state), ptr(x), x.stride(0), x.shape[0], ptr(row_tok), ptr(row_seq),
+                                ptr(row_slot), ptr(row_back), ptr(blk_tab), n_blk, ptr(chunk_tab), 0 if chunk_tab is None else chunk_tab.shape[0],
+                                max_len, flags, ptr(out), ptr(trace), ptr(ws), ws.numel(), current_stream()), "mn_hyb_step")
+
+
+class MultiStreamSteps(NativeSteps):
+    """Passes on the multi-stream step function (mn_ms_step): `struct` = the decoder's MsModel."""
+    STATE_KEYS = ("k", "v")
+    STATE_STRUCT = _lib.MsState
+
+    def _workspace_bytes(self, rows, max_len):
+        return lib().mn_ms_workspace_bytes(C.byref(self.struct), rows)
+
+    def _launch(self, x, row_tok, row_seq, row_slot, row_back, blk_tab, n_blk, chunk_tab, max_len, flags, out, trace, ws):
+        check(lib().mn_ms_step(C.byref(self.struct), C.byref(self.state), ptr(x), x.stride(0), x.shape[0], ptr(row_seq), ptr(row_slot), ptr(blk_tab),
+                               n_blk, max_len, flags, ptr(out), ptr(trace), ptr(ws), ws.numel(), current_stream()), "mn_ms_step")
 
 
 class DecodeGraph:
