@@ -134,15 +134,18 @@ def attention_mixer(h, sd, p, m, eps, v_first):
 
 
 # ---- experts -------------------------------------------------------------------------------------------------------------------
-def pick_experts(h, w_router, top):
-    """-> (experts [T, top], their scores [T, top])."""
-    s = torch.sigmoid(h @ f64(w_router).T)
-    idx = torch.argsort(s, dim=-1, descending=True, stable=True)[:, :top]
-    return idx, torch.gather(s, 1, idx)
+def pick_experts(h, w_router, top, gaps=None):
+    """-> (experts [T, top], their scores [T, top]); gaps: a list that receives the distance [T] of the chosen logits from the next one."""
+    z = h @ f64(w_router).T
+    idx = torch.argsort(z, dim=-1, descending=True, stable=True)[:, :top]
+    if gaps is not None and top < z.shape[1]:
+        best = torch.topk(z, top + 1, dim=-1).values
+        gaps.append(best[:, top - 1] - best[:, top])
+    return idx, torch.sigmoid(torch.gather(z, 1, idx))
 
 
-def expert_mixture(h, sd, p, mlp):
-    idx, w = pick_experts(h, sd[p + "router"], int(mlp["router"]["top"]))
+def expert_mixture(h, sd, p, mlp, gaps=None):
+    idx, w = pick_experts(h, sd[p + "router"], int(mlp["router"]["top"]), gaps)
     y = torch.zeros_like(h)
     for e in range(int(mlp["router"]["experts"])):
         gate, up, down = (f64(sd[f"{p}e{e}.{n}"]) for n in ("gate", "up", "down"))
@@ -155,8 +158,8 @@ def expert_mixture(h, sd, p, mlp):
 
 
 # ---- the model -----------------------------------------------------------------------------------------------------------------
-def forward(cfg, sd, tokens):
-    """-> (logits [T, vocab], the streams' sum after every layer [layers, T, width])."""
+def forward(cfg, sd, tokens, gaps=None):
+    """-> (logits [T, vocab], the streams' sum after every layer [layers, T, width]); gaps as in pick_experts, one entry per routed layer."""
     eps = float(cfg["norm"]["eps"])
     x = f64(sd["embed"])[torch.as_tensor(tokens, dtype=torch.long)] * float((cfg.get("embedding") or {}).get("scale", 1.0))
     X = torch.stack([x] * int(cfg["streams"]))
@@ -170,6 +173,93 @@ def forward(cfg, sd, tokens):
         X = streams_write(X, y, sd[p + "hc1.mix"], sd[p + "hc1.out"])
         if ly.get("mlp") is not None:
             h = norm_zero(streams_read(X, sd[p + "hc2.in"]), sd[p + "norm2"], eps)
-            X = streams_write(X, expert_mixture(h, sd, p + "mlp.", ly["mlp"]), sd[p + "hc2.mix"], sd[p + "hc2.out"])
+            X = streams_write(X, expert_mixture(h, sd, p + "mlp.", ly["mlp"], gaps), sd[p + "hc2.mix"], sd[p + "hc2.out"])
         trace.append(X.sum(0))
     return norm_zero(X.sum(0), sd["final.norm"], eps) @ f64(sd["embed"]).T, torch.stack(trace)
+
+
+# ---- small models for the tests ----------------------------------------------------------------------------------------------------
+def moe(experts, top, ff):
+    return {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff}}
+
+
+def attention_layer(heads=4, kv_heads=2, dim=16, vdim=12, scale=0.3, rot=(10000.0, 8), scaling=(4.0, 64, 8.0, 1.0), chunk=11, v_mix=True, mlp=None):
+    m = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=scale)
+    if rot:
+        m["rot"] = {"base": rot[0], "dims": rot[1]}
+        if scaling:
+            m["rot"]["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+    if chunk:
+        m["mask"] = {"size": chunk}
+    if v_mix:
+        m["v_mix"] = True
+    return {"type": "attention", "mixer": m, "mlp": mlp}
+
+
+def small_config(layers, width=64, vocab=80, streams=3, scale=2.5, eps=1e-5):
+    return {"architecture": "Fegarax", "width": width, "vocab": vocab, "streams": streams, "norm": {"eps": eps}, "embedding": {"scale": scale},
+            "layers": layers}
+
+
+def param_shapes(cfg):
+    W, V, S = cfg["width"], cfg["vocab"], cfg["streams"]
+    s = {"embed": (V, W), "final.norm": (W,)}
+    for i, ly in enumerate(cfg["layers"]):
+        p, m, mlp = f"l{i}.", ly["mixer"], ly.get("mlp")
+        nq, nk, nv, no = (m[a] * m[b] for a, b in (("heads", "dim"), ("kv_heads", "dim"), ("kv_heads", "vdim"), ("heads", "vdim")))
+        for n, rows in (("q", nq), ("k", nk), ("v", nv)):
+            s.update({f"{p}mix.{n}": (rows, W), f"{p}mix.{n}.b": (rows,)})
+        s.update({p + "norm1": (W,), p + "mix.q.norm": (nq,), p + "mix.k.norm": (nk,), p + "mix.g": (no, W), p + "mix.o": (W, no)})
+        if m.get("v_mix"):
+            s[p + "mix.vmix"] = ()
+        if mlp is not None:
+            ff = mlp["expert"]["ff"]
+            for j in range(mlp["router"]["experts"]):
+                s.update({f"{p}mlp.e{j}.gate": (ff, W), f"{p}mlp.e{j}.up": (ff, W), f"{p}mlp.e{j}.down": (W, ff)})
+            s.update({p + "norm2": (W,), p + "mlp.router": (mlp["router"]["experts"], W)})
+        for q in (1, 2) if mlp is not None else (1,):
+            s.update({f"{p}hc{q}.in": (S,), f"{p}hc{q}.out": (S,), f"{p}hc{q}.mix": (S, S)})
+    return s
+
+
+def random_weights(cfg, seed=0):
+    """bf16 tensors under the checkpoint's names.  The streams read, mix and take results unequally; experts' scores lie well apart."""
+    g = torch.Generator().manual_seed(seed)
+    sd = {}
+    for k, shp in param_shapes(cfg).items():
+        r = torch.randn(shp, generator=g)
+        if k == "embed":
+            t = r
+        elif k.endswith((".q.norm", ".k.norm")):
+            t = 1.0 + 0.2 * r
+        elif k.endswith((".norm1", ".norm2", "final.norm")):
+            t = 0.2 * r
+        elif k.endswith(".b"):
+            t = 0.3 * r
+        elif k.endswith(".vmix"):
+            t = 0.4 + 0.2 * r
+        elif ".hc" in k and k.endswith(".mix"):
+            t = 0.7 * torch.eye(shp[0]) + 0.3 * r
+        elif ".hc" in k:
+            t = 0.5 + 0.4 * r
+        elif k.endswith(".router"):
+            t = 2.5 * r * shp[-1] ** -0.5
+        else:
+            t = 1.3 * r * shp[-1] ** -0.5
+        sd[k] = t.to(torch.bfloat16)
+    return sd
+
+
+def clear_tokens(cfg, sd, n, seed=1, gap=0.06):
+    """n random tokens none of which has a close call between experts (a chosen logit and the next one less than `gap` apart): rounding in
+    the products before a router must not change what it picks.  A token that has one is drawn again; the tokens before it do not depend on it."""
+    g = torch.Generator().manual_seed(seed)
+    t = torch.randint(0, cfg["vocab"], (n,), generator=g).tolist()
+    for _ in range(20 * n):
+        gaps = []
+        forward(cfg, sd, t, gaps)
+        close = (torch.stack(gaps).amin(0) < gap).nonzero() if gaps else []
+        if len(close) == 0:
+            return t
+        t[int(close[0])] = int(torch.randint(0, cfg["vocab"], (1,), generator=g))
+    raise RuntimeError("no tokens without close calls")
