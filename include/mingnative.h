@@ -1415,7 +1415,9 @@ MN_API int mn_talk_attn(const float* q, int64_t ldq, const float* k_arena, int64
 /* One launch between two sublayers, per row m: y = y[m] (optional) + sum_j ew_j ye[r(m, j)] (top > 0; r as in mn_moe_combine_residual, ew NULL:
  * every weight 1); with mix: x_t <- sum_s mix[s, t] x_s + out[t] y, stored to dst when given (in place allowed: dst = src); then
  * u = sum_s in[s] x_s (in NULL: the streams' sum) and, with w, u / sqrt(mean(u^2) + eps) * w (one_plus: * (1 + w)), to h (fp32) and / or
- * h16 (bf16).  Stream s of row m starts at src + m src_row + s src_stream (src_stream 0: all streams are the same row). */
+ * h16 (bf16; h16_lo: what the bf16 value leaves, bf16, same stride).  Stream s of row m starts at src + m src_row + s src_stream (src_stream 0:
+ * all streams are the same row).  ye_slabs > 1: ye is the sum of that many slabs, ye_slab values apart.  router (mn_streams_router_ok): the
+ * normed row times bf16 [experts, n] in fp32; the `picks` largest logits' indices and sigmoids go to idx / pw [M, picks]. */
 typedef struct mn_streams_args {
   const float* src; int64_t src_row, src_stream;
   float* dst;                                      /* [M, S, n] or NULL */
@@ -1429,9 +1431,18 @@ typedef struct mn_streams_args {
   float eps;
   float* h; int64_t ldh;
   uint16_t* h16; int64_t ldh16;
+  uint16_t* h16_lo;
+  int64_t ye_slab; int32_t ye_slabs;
+  int32_t experts;
+  const uint16_t* router;
+  int32_t* idx; float* pw;
+  int32_t picks;
 } mn_streams_args;
 MN_API size_t mn_sizeof_streams_args(void);
 MN_API int mn_streams_update_norm(const mn_streams_args* a, int M, void* stream);
+/* 1: rows, streams and router fit the form of the update that routes (at most 4 streams, n a multiple of 8 up to 8192, 512 experts with up to
+ * 64 rows and 16 with more).  Slabs and low parts with a router: up to 64 rows. */
+MN_API int mn_streams_router_ok(int M, int S, int n, int experts, const uint16_t* router);
 /* mn_proj_norm_rope_append with cos and sin multiplied by rot_mag, and with values that are mixed: v_keep (optional, fp32 [M, kv_heads vdim])
  * receives the row's values as projected; v_first (optional): v <- (1 - v_lambda) v + v_lambda v_first before the append. */
 MN_API int mn_proj_norm_rope_mix_append(const float* qkv, int64_t ldqkv, int M, int H, int G, int dim, int vdim, const uint16_t* q_norm,
@@ -1461,6 +1472,8 @@ MN_API int mn_gemm256_grouped_tiles_scaled(const uint16_t* A, int64_t lda, int64
                                            const float* row_scale, void* C, int64_t ldc, int64_t c_lo_off, int N, int K, int epi, void* stream);
 MN_API int mn_silu_mul_rows_scaled(const float* x, int64_t ldx, const float* x_scale, float* y, int64_t ldy, uint16_t* y16, int64_t ldy16, int M,
                                    int n, void* stream);
+/* P fp32 [nz][M][2 n] (slabs of the grouped weight-streaming product) -> y bf16 [2][M][n], high rows then low rows, of silu(s gate) * (s up) */
+MN_API int mn_silu_split_rows_scaled(const float* P, int nz, int M, int n, const float* x_scale, uint16_t* y, void* stream);
 MN_API int mn_gemv_glu_indexed_scaled(const float* A, int64_t lda, int a_div, const uint16_t* W, int64_t ldw, int64_t w_bs, const int32_t* w_idx,
                                       int n_idx, const float* x_scale, float* C, int64_t ldc, int Z, int N, int K, void* stream);
 

@@ -196,7 +196,9 @@ class StreamsArgs(C.Structure):
     _fields_ = [("src", C.c_void_p), ("src_row", C.c_int64), ("src_stream", C.c_int64), ("dst", C.c_void_p), ("S", C.c_int32), ("n", C.c_int32),
                 ("mix", C.c_void_p), ("out", C.c_void_p), ("in_", C.c_void_p), ("y", C.c_void_p), ("ldy", C.c_int64), ("ye", C.c_void_p),
                 ("ldye", C.c_int64), ("slot_of", C.c_void_p), ("ew", C.c_void_p), ("top", C.c_int32), ("one_plus", C.c_int32),
-                ("w", C.c_void_p), ("eps", C.c_float), ("h", C.c_void_p), ("ldh", C.c_int64), ("h16", C.c_void_p), ("ldh16", C.c_int64)]
+                ("w", C.c_void_p), ("eps", C.c_float), ("h", C.c_void_p), ("ldh", C.c_int64), ("h16", C.c_void_p), ("ldh16", C.c_int64),
+                ("h16_lo", C.c_void_p), ("ye_slab", C.c_int64), ("ye_slabs", C.c_int32), ("experts", C.c_int32), ("router", C.c_void_p),
+                ("idx", C.c_void_p), ("pw", C.c_void_p), ("picks", C.c_int32)]
 
 
 class MsLayer(C.Structure):
@@ -470,6 +472,8 @@ SYMBOLS = {
     # section 14: multi-stream sequence models
     "mn_sizeof_streams_args": (_sz, []), "mn_sizeof_ms_layer": (_sz, []), "mn_sizeof_ms_model": (_sz, []), "mn_sizeof_ms_state": (_sz, []),
     "mn_streams_update_norm": (_i, [C.POINTER(StreamsArgs), _i, _p]),
+    "mn_streams_router_ok": (_i, [_i, _i, _i, _i, _p]),
+    "mn_silu_split_rows_scaled": (_i, [_p, _i, _i, _i, _p, _p, _p]),
     "mn_proj_norm_rope_mix_append": (_i, [_p, _i64, _i, _i, _i, _i, _i, _p, _p, _f, _i, _i, _p, _f, _f, _p, _i64, _p, _i64, _f, _p, _p, _p, _i64, _p,
                                           _i64, _p, _i64, _i, _p]),
     "mn_window_pool_attn_blocks_gate": (_i, [_p, _i64, _p, _i64, _p, _i64, _p, _p, _p, _f, _i, _p, _i64, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i,

@@ -195,7 +195,7 @@ extern "C" int mn_struct_layout(int which, size_t* offsets, int cap) {
   static const size_t streams[] = {
 #define F(f) MN_OFF(mn_streams_args, f)
       F(src) F(src_row) F(src_stream) F(dst) F(S) F(n) F(mix) F(out) F(in) F(y) F(ldy) F(ye) F(ldye) F(slot_of) F(ew) F(top) F(one_plus) F(w)
-      F(eps) F(h) F(ldh) F(h16) F(ldh16)
+      F(eps) F(h) F(ldh) F(h16) F(ldh16) F(h16_lo) F(ye_slab) F(ye_slabs) F(experts) F(router) F(idx) F(pw) F(picks)
 #undef F
   };
   static const size_t ms_layer[] = {

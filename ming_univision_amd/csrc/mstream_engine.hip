@@ -6,10 +6,12 @@
 //   whole-projection norms, rotation, value mixing, append; the block attention over the row's chunk / window, the heads' sinks in
 //   the denominator, the output gate in its epilogue; W_o
 //   h = norm(sum_s in2[s] x_s)
-//   router -> picks and weights; experts fed with weight * h: the weight scales the gate and up products
+//   router -> picks and weights (few rows or few experts: in the launch that norms); experts fed with weight * h: the weight scales the gate and up products
 // Matrix products go through the routing of seq_linear.h; the experts run
-//   MN_SEQ_ARITH_BF16, M > 8    sorted by expert on a grouped bf16 MFMA GEMM: the 256 x 256-tile kernel over the list of live row tiles when
-//                               width and expert width are multiples of 64, else the 128-tile kernel when they are multiples of 8
+//   MN_SEQ_ARITH_BF16, M > 64      sorted by expert on a grouped bf16 MFMA GEMM: the 256 x 256-tile kernel over the list of live row tiles when
+//                                  width and expert width are multiples of 64, else the 128-tile kernel when they are multiples of 8
+//   MN_SEQ_ARITH_BF16, 9 .. 64     sorted by expert on the grouped weight-streaming MFMA product (bf16 hi / lo rows): every chosen expert's
+//                                  weights once; its slabs are summed by the activation's launch and by the next read of the streams
 //   otherwise                   one (row, pick) pair at a time against the weights its index names (fp32 FMA)
 #include "seq_linear.h"
 
@@ -18,6 +20,8 @@ extern "C" size_t mn_sizeof_ms_model(void) { return sizeof(mn_ms_model); }
 extern "C" size_t mn_sizeof_ms_state(void) { return sizeof(mn_ms_state); }
 
 namespace {
+
+constexpr int STREAM_SLABS = 2;      // most K-range slabs of a grouped weight-streaming product (mn_stream_mfma_grouped_slices)
 
 inline int pad8(int n) { return (n + 7) / 8 * 8; }
 
@@ -39,12 +43,13 @@ struct MPlan {
   size_t gemm_ws = 0, attn_ws = 0;
 };
 
-enum { EXPERTS_INDEXED = 0, EXPERTS_GROUPED = 1, EXPERTS_TILES = 2 };
+enum { EXPERTS_INDEXED = 0, EXPERTS_GROUPED = 1, EXPERTS_TILES = 2, EXPERTS_STREAM = 3 };
 int expert_route(const mn_ms_model* m, const mn_ms_layer& l, int M) {
   if (m->arith != MN_SEQ_ARITH_BF16 || M <= 8 || l.experts > 128 || (int64_t)M * l.top > 65536 ||
       ((((uintptr_t)l.w_gate_up) | ((uintptr_t)l.w_down)) & 15) != 0)
     return EXPERTS_INDEXED;
   const int64_t W = m->width, ff = l.expert_ff;
+  if (M <= 64 && (W % 8) == 0 && (ff % 8) == 0) return EXPERTS_STREAM;
   if ((W % 64) == 0 && (ff % 64) == 0 && 2 * ff * W * 2 < ((int64_t)1 << 32) && (int64_t)M * l.top * (W > ff ? W : ff) * 2 < ((int64_t)1 << 32))
     return EXPERTS_TILES;
   if ((W % 8) == 0 && (ff % 8) == 0) return EXPERTS_GROUPED;
@@ -80,10 +85,10 @@ MPlan make_plan(const mn_ms_model* m, int M) {
 extern "C" size_t mn_ms_workspace_bytes(const mn_ms_model* m, int M) {
   if (!m || !m->layers || M < 1) return 0;
   const MPlan p = make_plan(m, M);
-  const size_t W = m->width, R = (size_t)M, Z = R * p.top;
+  const size_t W = m->width, R = (size_t)M, Z = R * p.top, few = M <= 64 ? STREAM_SLABS : 1;       // few rows: hi / lo rows, slabs
   size_t n = 0;
   n += al(R * m->streams * W * 4);                     // the streams
-  n += al(R * W * 4) + al(R * W * 2);                  // normed rows + bf16
+  n += al(R * W * 4) + al(few * R * W * 2);            // normed rows + bf16
   n += al(R * p.n_in * 4);                             // stacked input projections
   n += al(R * p.cq * 4);                               // queries
   n += al(R * p.cv * 4);                               // the values later layers mix in
@@ -91,9 +96,9 @@ extern "C" size_t mn_ms_workspace_bytes(const mn_ms_model* m, int M) {
   n += al(R * W * 4);                                  // sublayer result
   n += al(R * p.n_router * 4);                         // router logits
   n += al(Z * 4) + 2 * al(Z * 4);                      // chosen experts; weights, weights in the sorted order
-  n += al(Z * 2 * p.ff * 4);                           // [gate ; up] of the pairs
-  n += al(Z * p.ff * 4) + al(Z * p.ff * 2);            // their activation + bf16
-  n += al(Z * W * 4);                                  // their results
+  n += al(few * Z * 2 * p.ff * 4);                     // [gate ; up] of the pairs
+  n += al(Z * p.ff * 4) + al(few * Z * p.ff * 2);      // their activation + bf16
+  n += al(few * Z * W * 4);                            // their results
   n += al(Z * W * 2);                                  // gathered bf16 rows
   n += 2 * al(((size_t)p.experts + 1) * 4) + 2 * al(Z * 4);   // counts, offsets, perm, slot_of
   n += 2 * al((Z / 256 + p.experts + 1) * 4) + al(4);         // live row tiles of the grouped products, their count
@@ -114,14 +119,14 @@ extern "C" int mn_ms_step(const mn_ms_model* m, const mn_ms_state* st, const flo
   if (one_row) n_blk = M;
   const MPlan p = make_plan(m, M);
   const int W = m->width, S = m->streams, arith = m->arith;
-  const size_t R = (size_t)M, Zmax = R * p.top;
+  const size_t R = (size_t)M, Zmax = R * p.top, few = M <= 64 ? STREAM_SLABS : 1;
   MN_CHECK_ARG(Zmax <= 65535, "mn_ms_step: %d rows x %d picks exceed 65535 (row, expert) pairs per step", M, p.top);
   const bool want16 = arith == MN_SEQ_ARITH_BF16 && M > 64;       // bf16 copies feed the tiled MFMA GEMMs only
   char* wp = reinterpret_cast<char*>(workspace);
   auto take = [&](size_t bytes) { char* q = wp; wp += al(bytes); return q; };
   float* xs = (float*)take(R * S * W * 4);
   float* hf = (float*)take(R * W * 4);
-  uint16_t* hh = (uint16_t*)take(R * W * 2);
+  uint16_t* hh = (uint16_t*)take(few * R * W * 2);
   float* pin = (float*)take(R * p.n_in * 4);
   float* qf = (float*)take(R * p.cq * 4);
   float* vfirst = (float*)take(R * p.cv * 4);
@@ -132,10 +137,10 @@ extern "C" int mn_ms_step(const mn_ms_model* m, const mn_ms_state* st, const flo
   int32_t* tidx = (int32_t*)take(Zmax * 4);
   float* tw = (float*)take(Zmax * 4);
   float* tws = (float*)take(Zmax * 4);
-  float* gu = (float*)take(Zmax * 2 * p.ff * 4);
+  float* gu = (float*)take(few * Zmax * 2 * p.ff * 4);
   float* ea = (float*)take(Zmax * p.ff * 4);
-  uint16_t* eah = (uint16_t*)take(Zmax * p.ff * 2);
-  float* ye = (float*)take(Zmax * W * 4);
+  uint16_t* eah = (uint16_t*)take(few * Zmax * p.ff * 2);
+  float* ye = (float*)take(few * Zmax * W * 4);
   uint16_t* xg = (uint16_t*)take(Zmax * W * 2);
   int32_t* counts = (int32_t*)take(((size_t)p.experts + 1) * 4);
   int32_t* offsets = (int32_t*)take(((size_t)p.experts + 1) * 4);
@@ -157,13 +162,17 @@ extern "C" int mn_ms_step(const mn_ms_model* m, const mn_ms_state* st, const flo
   sa.src = x; sa.src_row = ldx; sa.src_stream = 0;
   sa.S = S; sa.n = W; sa.eps = m->eps; sa.one_plus = m->norm_one_plus;
   // the streams take what is pending; sum_s in[s] x_s, normed with w (NULL: as it is), goes to h / h16
-  auto streams_stage = [&](const float* in, const uint16_t* w, float* h, uint16_t* h16) -> int {
+  // and, with a router, its picks and scores to tidx / tw; hi_lo: h16 holds the low parts behind its M rows
+  struct Route { const uint16_t* w; int experts, picks; };
+  auto streams_stage = [&](const float* in, const uint16_t* w, float* h, uint16_t* h16, const Route* r = nullptr, bool hi_lo = false) -> int {
     mn_streams_args a = sa;
     a.dst = a.mix ? xs : nullptr;
     a.in = in; a.w = w; a.h = h; a.ldh = W; a.h16 = h16; a.ldh16 = W;
+    if (hi_lo) a.h16_lo = h16 + R * W;
+    if (r) { a.router = r->w; a.experts = r->experts; a.picks = r->picks; a.idx = tidx; a.pw = tw; }
     const int rc2 = mn_streams_update_norm(&a, M, stream);
     if (a.dst) { sa.src = xs; sa.src_row = (int64_t)S * W; sa.src_stream = W; }
-    sa.mix = sa.out = nullptr; sa.y = sa.ye = nullptr; sa.slot_of = nullptr; sa.ew = nullptr; sa.top = 0;
+    sa.mix = sa.out = nullptr; sa.y = sa.ye = nullptr; sa.slot_of = nullptr; sa.ew = nullptr; sa.top = 0; sa.ye_slabs = 0;
     return rc2;
   };
   bool have_first = false;
@@ -203,15 +212,19 @@ extern "C" int mn_ms_step(const mn_ms_model* m, const mn_ms_state* st, const flo
     // ---- experts ----
     if (E > 0) {
       const int route = expert_route(m, l, M);
-      const bool h16_only = hh && mfma_ok(l.w_router, W) && route != EXPERTS_INDEXED;
-      MN_TRY(streams_stage(l.hc2_in, l.norm2, h16_only ? nullptr : hf, hh));
-      MN_TRY(linear(arith, M, hf, W, hh, W, l.w_router, d.n_router, W, nullptr, rl, d.n_router, gws, gwb, stream));
-      MN_TRY(mn_router_sigmoid_topk_rows(rl, d.n_router, M, E, top, tidx, tw, stream));
-      const uint16_t* h16 = hh;
-      if (route != EXPERTS_INDEXED && !h16) {          // few rows: the sublayer input was written in fp32 only
-        MN_TRY(mn_f32_to_bf16(hf, hh_buf, (int64_t)M * W, stream));
-        h16 = hh_buf;
+      const bool stream_rows = route == EXPERTS_STREAM;
+      const bool ride = mn_streams_router_ok(M, S, W, E, l.w_router) && (((uintptr_t)sa.src) & 15) == 0 && (sa.src_row % 4) == 0;
+      if (ride) {
+        const Route r{l.w_router, E, top};
+        MN_TRY(streams_stage(l.hc2_in, l.norm2, route == EXPERTS_INDEXED ? hf : nullptr, route == EXPERTS_INDEXED ? nullptr : hh_buf, &r, stream_rows));
+      } else {
+        const bool h16_only = hh && mfma_ok(l.w_router, W) && route != EXPERTS_INDEXED;
+        uint16_t* const h16 = route == EXPERTS_INDEXED ? hh : hh_buf;
+        MN_TRY(streams_stage(l.hc2_in, l.norm2, h16_only ? nullptr : hf, h16, nullptr, stream_rows));
+        MN_TRY(linear(arith, M, hf, W, hh, W, l.w_router, d.n_router, W, nullptr, rl, d.n_router, gws, gwb, stream));
+        MN_TRY(mn_router_sigmoid_topk_rows(rl, d.n_router, M, E, top, tidx, tw, stream));
       }
+      const uint16_t* h16 = hh_buf;
       const int32_t* so = nullptr;
       if (route == EXPERTS_TILES) {
         const int max_mtiles = Z / 256 + E;
@@ -220,6 +233,15 @@ extern "C" int mn_ms_step(const mn_ms_model* m, const mn_ms_state* st, const flo
                                                max_mtiles, tws, eah, ff, 0, ff, W, 6, stream));
         MN_TRY(mn_gemm256_grouped_tiles(eah, ff, 0, Z, nullptr, l.w_down, ff, (int64_t)W * ff, offsets, counts, E, tile_g, tile_m0, n_tiles,
                                         max_mtiles, ye, W, 0, W, ff, 0, stream));
+        so = slot_of;
+      } else if (route == EXPERTS_STREAM) {
+        MN_TRY(mn_moe_sort_weights(tidx, tw, M, top, E, counts, offsets, perm, slot_of, tws, 0, nullptr, nullptr, nullptr, stream));
+        const int nz = mn_stream_mfma_grouped(h16, M, l.w_gate_up, (int64_t)2 * ff * W, gu, Z, offsets, perm, E, M, 2 * ff, W, stream);
+        if (nz < 0) return nz;
+        MN_TRY(mn_silu_split_rows_scaled(gu, nz, Z, ff, tws, eah, stream));
+        const int nz2 = mn_stream_mfma_grouped(eah, Z, l.w_down, (int64_t)W * ff, ye, Z, offsets, nullptr, E, M, W, ff, stream);
+        if (nz2 < 0) return nz2;
+        sa.ye_slab = (int64_t)Z * W; sa.ye_slabs = nz2;
         so = slot_of;
       } else if (route == EXPERTS_GROUPED) {
         MN_TRY(mn_moe_sort_weights(tidx, tw, M, top, E, counts, offsets, perm, slot_of, tws, 0, nullptr, nullptr, nullptr, stream));

@@ -19,6 +19,7 @@
 
 #include "common.h"
 #include "mfma_f32_tiles.h"
+#include "router_device.h"
 
 extern "C" int mn_rotary_frequencies_host(int dims, double base, double factor, double original, double fast, double slow, float* freq,
                                           float* mag) {
@@ -994,9 +995,7 @@ __global__ __launch_bounds__(256) void mingru_pass3_kernel(MinGruArgs a) {
   }
 }
 
-// one wave per row: `top` rounds of arg-max (ties: the lower index), then the softmax over the chosen logits (SIGMOID: every chosen
-// logit's sigmoid as it is).  Lane l owns the
-// logits l, l + 64, ... and a bit per owned logit that says it has been chosen (E <= 4096).
+// one wave per row: wave_topk
 template <bool SIGMOID>
 __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restrict__ logits, int64_t ld, int M, int E, int top,
                                                           int32_t* __restrict__ idx, float* __restrict__ w, const float* __restrict__ sx,
@@ -1012,30 +1011,7 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restric
   const float* z = logits + (int64_t)row * ld;
   int32_t* ir = idx + (int64_t)row * top;
   float* wr = w + (int64_t)row * top;
-  uint64_t taken = 0;
-  float first = 0.f, sum = 0.f;
-  for (int k = 0; k < top; ++k) {
-    float best = -INFINITY;
-    int bi = 0x7fffffff;
-    for (int e = lane, i = 0; e < E; e += 64, ++i) {
-      const float v = z[e];
-      if (!((taken >> i) & 1) && (v > best || (v == best && e < bi) || bi == 0x7fffffff)) { best = v; bi = e; }
-    }
-    for (int off = 32; off >= 1; off >>= 1) {
-      const float ob = __shfl_xor(best, off);
-      const int oi = __shfl_xor(bi, off);
-      if (oi != 0x7fffffff && (bi == 0x7fffffff || ob > best || (ob == best && oi < bi))) { best = ob; bi = oi; }
-    }
-    if ((bi & 63) == lane) taken |= (uint64_t)1 << (bi >> 6);
-    if (k == 0) first = best;
-    const float p = SIGMOID ? sigmoid_f(best) : expf(best - first);
-    sum += p;
-    if (lane == 0) { ir[k] = bi; wr[k] = p; }
-  }
-  if (SIGMOID) return;
-  // lane 0 wrote the unnormalised weights and is the one that scales them
-  if (lane == 0)
-    for (int k = 0; k < top; ++k) wr[k] = wr[k] / sum;
+  wave_topk<SIGMOID>(z, E, top, lane, ir, wr);
 }
 
 __global__ __launch_bounds__(256) void silu_mul_kernel(const float* __restrict__ x, int64_t ldx, const float* __restrict__ s,

@@ -130,7 +130,7 @@ struct ProjNormArgs {
 template <int NT, int GW>
 __global__ __launch_bounds__(NT) void proj_norm_rope_append_kernel(ProjNormArgs a) {
   extern __shared__ __align__(16) float cs[];
-  __shared__ float red[NT / 64];
+  __shared__ float red[2 * (NT / 64)];
   typedef float vec_t __attribute__((ext_vector_type(4)));
   const int m = blockIdx.x, tid = threadIdx.x, half = a.rot_dims >> 1;
   const int nq = a.H * a.dim, nk = a.G * a.dim, nv = a.G * a.vdim;
@@ -154,9 +154,14 @@ __global__ __launch_bounds__(NT) void proj_norm_rope_append_kernel(ProjNormArgs 
     return ss;
   };
   float rq = 1.0f, rk = 1.0f;
-  if (a.q_norm) rq = 1.0f / sqrtf(block_sum(square_sum(row, nq), red) / (float)nq + a.eps);
-  if (a.k_norm) rk = 1.0f / sqrtf(block_sum(square_sum(row + nq, nk), red) / (float)nk + a.eps);
+  float sq = a.q_norm ? wave_sum(square_sum(row, nq)) : 0.f, sk = a.k_norm ? wave_sum(square_sum(row + nq, nk)) : 0.f;
+  if ((tid & 63) == 0) { red[tid >> 6] = sq; red[NT / 64 + (tid >> 6)] = sk; }
   __syncthreads();
+  sq = sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < NT / 64; ++i) { sq += red[i]; sk += red[NT / 64 + i]; }
+  if (a.q_norm) rq = 1.0f / sqrtf(sq / (float)nq + a.eps);
+  if (a.k_norm) rk = 1.0f / sqrtf(sk / (float)nk + a.eps);
   float* kd = a.k_arena + ((int64_t)seq * a.t_max + pos) * a.ldk;
   // one projection: n values at src with their norm weights (w NULL: none) to dst, times scale
   auto turn = [&](const float* src, int n, const bf16_t* w, float r, float scale, float* dst) {

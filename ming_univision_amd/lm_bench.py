@@ -35,6 +35,14 @@ recurrence — and its delta rule beside Daberax's: same width, depth, head coun
 gla - attention, once with dense feed-forwards of equal size (two matrices of 1.5 ff on both), once with 8 experts top-2 on both (three
 matrices of ff / 2; no shared expert).  Its attention sees chunks of 1024 tokens and is priced on the pairs it sees; the mixing of the
 heads' scores is not counted as work.  The recurrences are priced like the lightning recurrence and the delta rule.
+
+Fegarax (`--lm-model fegarax`: attention and experts in every layer, four residual streams) stands beside Zuzenex and Sabezen stacks of
+attention layers only: same width, depth, head counts and 128-wide heads, 8 experts top-2 of equal parameter count on all three (three
+matrices of ff / 2 against Zuzenex' two of 3/4 ff), no shared expert.  Fegarax and Sabezen see chunks of 1024 tokens, Zuzenex every earlier
+token.  Its attention (with the output gate) runs on Zuzenex' kernel; its stream update stands beside Sabezen's residual sum with expert
+combine and LayerNorm, both priced on the bytes they must move; the experts' products with a factor per row beside those without,
+priced on their multiply-adds (prompts) or on the weight bytes of the experts that are chosen (decode rows).  Short kernels are
+timed as a captured graph of launches.
 """
 import sys
 import time
@@ -60,6 +68,59 @@ def _time(fn, iters, warm=2):
         fn()
     torch.cuda.synchronize()
     return (time.perf_counter() - t0) / iters
+
+
+def _time_graph(fn, n=20, iters=5):
+    """Seconds of one fn() whose launches are too short for the host: n calls captured as a graph."""
+    torch.cuda.synchronize()                                 # the side stream does not wait for what the current one still writes
+    side = torch.cuda.Stream()
+    with torch.cuda.stream(side):
+        fn()
+    side.synchronize()
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        for _ in range(n):
+            fn()
+    return _time(g.replay, iters) / n
+
+
+def _rates(dec, s, T, batches, n_dec):
+    """Prefill and decode tokens/s of a decoder on the serving path: one prompt of T tokens, then lock-step decode steps of B sequences that
+    all continue it, launched one by one and replayed from the captured step."""
+    from ._lib import check, current_stream, lib, ptr
+    dev = dec.device
+    ids = torch.randint(0, s["vocab"], (T,), device=dev)
+    x = dec.embed(ids)
+    out = {"prefill_tokens_per_s": T / _time(lambda: dec.forward_spans(x, [(0, T, 0)], tokens=ids), 3)}
+    for B in batches:
+        for ly in dec.state_t:
+            for t in ly.values():
+                if t is not None and B > 1:
+                    t[1:B].copy_(t[0:1].expand_as(t[1:B]))
+        row_seq = torch.arange(B, dtype=torch.int32, device=dev)
+        back, blk = dec.decode_tables(B)
+        tok = torch.randint(0, s["vocab"], (B,), device=dev)
+        xb, tok32 = dec.embed(tok), tok.to(torch.int32)
+        more = dict(row_tok=tok32) if dec.needs_tokens else {}
+
+        def loop():
+            slot = torch.full((B,), T, dtype=torch.int32, device=dev)
+            ln = slot + 1
+            for i in range(n_dec):
+                dec.step(xb, row_seq, slot, back, ln, blk, T + i + 1, distinct=True, **more)
+                check(lib().mn_rows_advance(ptr(slot), ptr(ln), None, B, 1, current_stream()), "mn_rows_advance")
+        out[f"decode_b{B}_tokens_per_s"] = B * n_dec / _time(loop, 2, 1)
+        slot_g = torch.full((B,), T, dtype=torch.int32, device=dev)
+        ln_g = slot_g + 1
+        graph = dec.decode_graph(row_seq, slot_g, ln_g)
+
+        def loop_graph():
+            slot_g.fill_(T)
+            ln_g.fill_(T + 1)
+            for i in range(n_dec):
+                graph.run(xb, T + i + 1, tokens=tok32)
+        out[f"decode_b{B}_graph_tokens_per_s"] = B * n_dec / _time(loop_graph, 2, 1)
+    return out
 
 
 def pizitar_config(s):
@@ -234,54 +295,27 @@ def run_sakinex(s, T, batches, n_dec):
     return out
 
 
-def zuzenex_config(s, dense=False):
+def zuzenex_config(s, dense=False, attention_only=False):
     from .configuration import ZuzenexConfig
     H = s["heads"]
     mlp = dict(kind="moe", router=dict(experts=8, top=2, identity=1), expert=dict(ff=s["ff"] * 3 // 4), shared=dict(ff=s["ff"] * 3 // 4))
     if dense:
         mlp = dict(kind="dense", ff=s["ff"] * 3 // 2)
+    elif attention_only:                                     # beside models without a shared expert
+        mlp = dict(kind="moe", router=dict(experts=8, top=2, identity=0), expert=dict(ff=s["ff"] * 3 // 4))
     att = dict(type="attention", mixer=dict(heads=H, kv_heads=H // 4, dim=128, vdim=128, scale=128 ** -0.5, q_temp=dict(coef=0.1, every=1024)), mlp=mlp)
     lin = dict(type="lightning", mixer=dict(heads=H, dim=128, vdim=128, decay=[1.0 - 2.0 ** (-5 - 4 * h / H) for h in range(H)]), mlp=mlp)
-    order = [att, lin, lin, att]
+    order = [att] * 4 if attention_only else [att, lin, lin, att]
     return ZuzenexConfig(width=s["width"], vocab=s["vocab"], layers=[order[i % 4] for i in range(s["layers"])], norm=dict(eps=1e-6))
 
 
-def run_zuzenex(s, T, batches, n_dec, dense=False):
+def run_zuzenex(s, T, batches, n_dec, dense=False, attention_only=False):
     from ._lib import check, current_stream, lib, ptr
     from .sequences import rows_of_spans
     from .zuzenex import ZuzenexDecoder
     dev = "cuda"
-    cfg = zuzenex_config(s, dense)
-    dec = ZuzenexDecoder.synthetic(cfg, dev, t_max=T + n_dec + 8, n_seq=max(batches), arith="bf16")
-    ids = torch.randint(0, s["vocab"], (T,), device=dev)
-    x = dec.embed(ids)
-    out = {"prefill_tokens_per_s": T / _time(lambda: dec.forward_spans(x, [(0, T, 0)]), 3)}
-    for B in batches:
-        for run in dec.state_t:                              # every sequence continues the prompt of sequence 0
-            for t in run.values():
-                if t is not None and B > 1:
-                    t[1:B].copy_(t[0:1].expand_as(t[1:B]))
-        row_seq = torch.arange(B, dtype=torch.int32, device=dev)
-        back, blk = dec.decode_tables(B)
-        xb = dec.embed(torch.randint(0, s["vocab"], (B,), device=dev))
-
-        def loop():
-            slot = torch.full((B,), T, dtype=torch.int32, device=dev)
-            ln = slot + 1
-            for i in range(n_dec):
-                dec.step(xb, row_seq, slot, back, ln, blk, T + i + 1, distinct=True)
-                check(lib().mn_rows_advance(ptr(slot), ptr(ln), None, B, 1, current_stream()), "mn_rows_advance")
-        out[f"decode_b{B}_tokens_per_s"] = B * n_dec / _time(loop, 2, 1)
-        slot_g = torch.full((B,), T, dtype=torch.int32, device=dev)
-        ln_g = slot_g + 1
-        graph = dec.decode_graph(row_seq, slot_g, ln_g)
-
-        def loop_graph():
-            slot_g.fill_(T)
-            ln_g.fill_(T + 1)
-            for i in range(n_dec):
-                graph.run(xb, T + i + 1)
-        out[f"decode_b{B}_graph_tokens_per_s"] = B * n_dec / _time(loop_graph, 2, 1)
+    dec = ZuzenexDecoder.synthetic(zuzenex_config(s, dense, attention_only), dev, t_max=T + n_dec + 8, n_seq=max(batches), arith="bf16")
+    out = _rates(dec, s, T, batches, n_dec)
     # the attention kernel alone, on the first run's arenas (an attention layer)
     H, G, d = s["heads"], s["heads"] // 4, 128
     st = dec.state_t[0]
@@ -309,6 +343,8 @@ def run_zuzenex(s, T, batches, n_dec, dense=False):
         t = _time(lambda: attn(B, row_seq, slot, 1), 20)
         byts = B * T * G * 2 * d * 4
         out[f"attn_decode_b{B}"] = dict(us=t * 1e6, gbs=byts / t / 1e9, of_peak=byts / t / 1e9 / HBM_GBS, key_splits=attn(B, row_seq, slot, 1))
+    if attention_only:
+        return out
     # the recurrence alone, on the second run's state (a lightning layer)
     lin = dec.state_t[1]["lin"]
     decay = torch.full((H,), 0.99, device=dev)
@@ -444,7 +480,7 @@ def run_daberax(s, T, batches, n_dec, window=1024):
 SABEZEN_CHUNK = 1024
 
 
-def sabezen_config(s, dense=True, chunk=SABEZEN_CHUNK):
+def sabezen_config(s, dense=True, chunk=SABEZEN_CHUNK, attention_only=False):
     from .configuration import SabezenConfig
     H = s["heads"]
     mlp = dict(kind="dense", ff=s["ff"] * 3 // 2) if dense else dict(kind="moe", router=dict(experts=8, top=2), expert=dict(ff=s["ff"] // 2))
@@ -452,7 +488,7 @@ def sabezen_config(s, dense=True, chunk=SABEZEN_CHUNK):
                                             mask=dict(size=chunk)), mlp=mlp)
     dlt = dict(type="channel_delta", mixer=dict(heads=H, kv_heads=H, dim=128, vdim=128, conv=4), mlp=mlp)
     gla = dict(type="gla", mixer=dict(heads=H, dim=128, vdim=128, tau=16.0), mlp=mlp)
-    order = [att, dlt, gla, att]
+    order = [att] * 4 if attention_only else [att, dlt, gla, att]
     return SabezenConfig(width=s["width"], vocab=s["vocab"], layers=[order[i % 4] for i in range(s["layers"])], norm=dict(eps=1e-6),
                          embedding=dict(scale=2.0))
 
@@ -463,37 +499,7 @@ def run_sabezen(s, T, batches, n_dec, dense=True, kernels=True):
     from .sequences import rows_of_spans
     dev = "cuda"
     dec = SabezenDecoder.synthetic(sabezen_config(s, dense), dev, t_max=T + n_dec + 8, n_seq=max(batches), arith="bf16")
-    ids = torch.randint(0, s["vocab"], (T,), device=dev)
-    x = dec.embed(ids)
-    out = {"prefill_tokens_per_s": T / _time(lambda: dec.forward_spans(x, [(0, T, 0)], tokens=ids), 3)}
-    for B in batches:
-        for ly in dec.state_t:                               # every sequence continues the prompt of sequence 0
-            for t in ly.values():
-                if t is not None and B > 1:
-                    t[1:B].copy_(t[0:1].expand_as(t[1:B]))
-        row_seq = torch.arange(B, dtype=torch.int32, device=dev)
-        back, blk = dec.decode_tables(B)
-        tok = torch.randint(0, s["vocab"], (B,), device=dev)
-        xb, tok32 = dec.embed(tok), tok.to(torch.int32)
-        more = dict(row_tok=tok32) if dec.needs_tokens else {}
-
-        def loop():
-            slot = torch.full((B,), T, dtype=torch.int32, device=dev)
-            ln = slot + 1
-            for i in range(n_dec):
-                dec.step(xb, row_seq, slot, back, ln, blk, T + i + 1, distinct=True, **more)
-                check(lib().mn_rows_advance(ptr(slot), ptr(ln), None, B, 1, current_stream()), "mn_rows_advance")
-        out[f"decode_b{B}_tokens_per_s"] = B * n_dec / _time(loop, 2, 1)
-        slot_g = torch.full((B,), T, dtype=torch.int32, device=dev)
-        ln_g = slot_g + 1
-        graph = dec.decode_graph(row_seq, slot_g, ln_g)
-
-        def loop_graph():
-            slot_g.fill_(T)
-            ln_g.fill_(T + 1)
-            for i in range(n_dec):
-                graph.run(xb, T + i + 1, tokens=tok32)
-        out[f"decode_b{B}_graph_tokens_per_s"] = B * n_dec / _time(loop_graph, 2, 1)
+    out = _rates(dec, s, T, batches, n_dec)
     if not kernels:
         return out
     # the kernels alone, on the layers' own arenas and states
@@ -559,6 +565,130 @@ def run_sabezen(s, T, batches, n_dec, dense=True, kernels=True):
     return out
 
 
+FEGARAX_CHUNK, FEGARAX_STREAMS = 1024, 4
+
+
+def fegarax_config(s):
+    from .configuration import FegaraxConfig
+    H = s["heads"]
+    att = dict(type="attention", mixer=dict(heads=H, kv_heads=H // 4, dim=128, vdim=128, scale=128 ** -0.5, v_mix=True, mask=dict(size=FEGARAX_CHUNK),
+                                            rot=dict(base=100000.0, dims=64, scaling=dict(factor=4.0, fast=32.0, original=4096, slow=1.0))),
+               mlp=dict(kind="moe", router=dict(experts=8, top=2), expert=dict(ff=s["ff"] // 2)))
+    return FegaraxConfig(width=s["width"], vocab=s["vocab"], layers=[att] * s["layers"], norm=dict(eps=1e-6), embedding=dict(scale=2.0),
+                         streams=FEGARAX_STREAMS)
+
+
+def run_fegarax(s, T, batches, n_dec):
+    from ._lib import StreamsArgs, check, current_stream, lib, ptr
+    from .fegarax import FegaraxDecoder
+    from .sequences import rows_of_spans
+    dev = "cuda"
+    dec = FegaraxDecoder.synthetic(fegarax_config(s), dev, t_max=T + n_dec + 8, n_seq=max(batches), arith="bf16")
+    out = _rates(dec, s, T, batches, n_dec)
+    H, G, d, W, S, ff, chunk = s["heads"], s["heads"] // 4, 128, s["width"], FEGARAX_STREAMS, s["ff"] // 2, FEGARAX_CHUNK
+    E, top = 8, 2
+    tabs = {k: torch.from_numpy(v).to(dev) for k, v in rows_of_spans([(0, T, 0)], dec.block_rows).items() if k != "max_len"}
+    st, L = dec.state_t[0], dec._layers[1]
+    n_in = (H + G) * d + G * d + H * d
+    pin, att = torch.randn(T, n_in, device=dev), torch.empty(T, H * d, device=dev)
+    q, vf = torch.randn(T, H * d, device=dev) * 0.05, torch.randn(T, G * d, device=dev)
+    aws = torch.empty(128 << 20, dtype=torch.uint8, device=dev)
+
+    def rows(B):
+        """Row arrays of a prompt (B None) or of a decode step at the context's end."""
+        if B is None:
+            return T, tabs["row_seq"], tabs["row_slot"], 0
+        return B, torch.arange(B, dtype=torch.int32, device=dev), torch.full((B,), T - 1, dtype=torch.int32, device=dev), 1
+
+    def attn(M, rs, rp, one_row):
+        n_blk = M if one_row else tabs["blk_tab"].shape[0]
+        ns = lib().mn_window_attn_splits(n_blk, H, G, one_row, chunk + 3)
+        check(lib().mn_window_pool_attn_blocks_gate(ptr(q), H * d, ptr(st["k"]), 0, ptr(st["v"]), 0, None, None, L.sink, 0.0, chunk,
+                                                    pin.data_ptr() + 4 * (n_in - H * d), n_in, ptr(rs), ptr(rp), None if one_row else ptr(tabs["blk_tab"]),
+                                                    n_blk, one_row, H, G, d, d, dec.t_max, 1, 0, 0, 1.0, ptr(att), H * d, None, 0, ns, ptr(aws),
+                                                    aws.numel(), -1, current_stream()), "mn_window_pool_attn_blocks_gate")
+        return ns
+
+    def record(name, t, byts=None, flops=None, peak=None, **kw):
+        out[name] = dict(us=t * 1e6, gbs=byts / t / 1e9, of_peak=byts / t / 1e9 / HBM_GBS, **kw) if flops is None else \
+            dict(us=t * 1e6, tflops=flops / t / 1e12, of_peak=flops / t / 1e12 / peak, **kw)
+    args = rows(None)
+    record("attn_prefill", _time(lambda: attn(*args), 5), flops=2 * 2 * H * d * sum(i % chunk + 1 for i in range(T)), peak=FMA_F32_TFLOPS,
+           on="fp32 MFMA", key_splits=attn(*args))
+    for B in batches:
+        args_b = rows(B)
+        record(f"attn_decode_b{B}", _time_graph(lambda: attn(*args_b)), byts=B * ((T - 1) % chunk + 1) * G * 2 * d * 4, key_splits=attn(*args_b))
+    # between two sublayers: the streams' update with the experts' results and the next norm; Sabezen's residual sum, combine and LayerNorm
+    X, y = torch.randn(T, S, W, device=dev), torch.randn(T, W, device=dev)
+    ye, h, h16 = torch.randn(T * top, W, device=dev), torch.empty(T, W, device=dev), torch.empty(T, W, dtype=torch.bfloat16, device=dev)
+    slot, ew = torch.randperm(T * top, device=dev).to(torch.int32), torch.rand(T * top, device=dev)
+    lnw = torch.ones(W, dtype=torch.bfloat16, device=dev)
+
+    def streams(M, experts, wide):
+        a = StreamsArgs(src=X.data_ptr(), src_row=S * W, src_stream=W, dst=X.data_ptr(), S=S, n=W, mix=L.hc1_mix, out=L.hc1_out, in_=L.hc2_in,
+                        y=None if experts else y.data_ptr(), ldy=W, ye=ye.data_ptr(), ldye=W, slot_of=slot.data_ptr() if wide else None,
+                        top=top if experts else 0, w=L.norm2, eps=1e-6, one_plus=1, h=None if wide else h.data_ptr(), ldh=W,
+                        h16=h16.data_ptr() if wide else None, ldh16=W)
+        check(lib().mn_streams_update_norm(a, M, current_stream()), "mn_streams_update_norm")
+
+    def residual(M, experts, wide):
+        check(lib().mn_add_layernorm_rows(ptr(X), W, None if experts else ptr(y), W, ptr(ye), W, ptr(slot) if wide else None, ptr(ew), 0.0,
+                                          top if experts else 0, ptr(lnw), 1e-6, None if wide else ptr(h), W, ptr(h16) if wide else None, W, M, W,
+                                          current_stream()), "mn_add_layernorm_rows")
+    for name, fn, copies in (("streams", streams, S), ("sabezen_residual_norm", residual, 1)):
+        for kind, experts in (("attn", False), ("experts", True)):
+            for B in (None,) + tuple(batches):
+                M, wide = B or T, B is None
+                byts = M * W * (copies * 8 + (top if experts else 1) * 4 + (2 if wide else 4))
+                record(f"{name}_{kind}_{'prefill' if wide else f'decode_b{B}'}", _time_graph(lambda: fn(M, experts, wide)), byts=byts)
+    # whole-projection norms, rotation, mixed values, append
+    for B in (None,) + tuple(batches):
+        M, rs, rp, _ = rows(B)
+        t = _time_graph(lambda: check(lib().mn_proj_norm_rope_mix_append(
+            ptr(pin), n_in, M, H, G, d, d, L.q_norm, L.k_norm, 1e-6, 64, 0, L.rot_freq, L.rot_mag, d ** -0.5, None, 0, ptr(vf), G * d, 0.4, ptr(rs), ptr(rp),
+            ptr(q), H * d, ptr(st["k"]), G * d, ptr(st["v"]), G * d, dec.t_max, current_stream()), "mn_proj_norm_rope_mix_append"))
+        record(f"append_{'prefill' if B is None else f'decode_b{B}'}", t, byts=M * 4 * (2 * (H + 2 * G) * d + G * d))
+    # the experts' products: a prompt's sorted pairs on the 256-tile kernel, decode rows pair by pair; with and without a factor per pair
+    Z = T * top
+    idx, pw = torch.stack([torch.randperm(E, device=dev)[:top] for _ in range(T)]).to(torch.int32).reshape(-1).contiguous(), torch.rand(Z, device=dev)
+    i32 = lambda n: torch.zeros(n, dtype=torch.int32, device=dev)  # noqa: E731
+    counts, offsets, perm, so, tg, tm, nt = i32(E + 1), i32(E + 1), i32(Z), i32(Z), i32(Z // 256 + E + 1), i32(Z // 256 + E + 1), i32(1)
+    ws, act, act16 = torch.empty(Z, device=dev), torch.empty(Z, ff, device=dev), torch.empty(Z, ff, dtype=torch.bfloat16, device=dev)
+    check(lib().mn_moe_sort_weights(ptr(idx), ptr(pw), T, top, E, ptr(counts), ptr(offsets), ptr(perm), ptr(so), ptr(ws), 256, ptr(tg), ptr(tm), ptr(nt),
+                                    current_stream()), "mn_moe_sort_weights")
+    for name, factor, pair in (("expert_gate_up", ws, pw), ("unscaled_gate_up", None, None)):
+        t = _time_graph(lambda: check(lib().mn_gemm256_grouped_tiles_scaled(
+            ptr(h16), W, 0, T, ptr(perm), L.w_gate_up, W, 2 * ff * W, ptr(offsets), ptr(counts), E, ptr(tg), ptr(tm), ptr(nt), Z // 256 + E, ptr(factor),
+            ptr(act16), ff, 0, ff, W, 6, current_stream()), "mn_gemm256_grouped_tiles_scaled"))
+        record(name + "_prefill", t, flops=2 * Z * 2 * ff * W, peak=MFMA_BF16_TFLOPS, on="bf16 MFMA")
+        t = _time_graph(lambda: check(lib().mn_gemv_glu_indexed_scaled(ptr(h), W, top, L.w_gate_up, W, 2 * ff * W, ptr(idx), E, ptr(pair), ptr(act), ff,
+                                                                       top, ff, W, current_stream()), "mn_gemv_glu_indexed_scaled"))
+        record(name + "_decode_b1", t, byts=top * 2 * ff * W * 2)
+    # 32 decode rows: the grouped weight-streaming product, and the 256-tile product the other decoders run at this size; every expert is chosen
+    B = 32
+    check(lib().mn_moe_sort_weights(ptr(idx), ptr(pw), B, top, E, ptr(counts), ptr(offsets), ptr(perm), ptr(so), ptr(ws), 256, ptr(tg), ptr(tm), ptr(nt),
+                                    current_stream()), "mn_moe_sort_weights")
+    hilo, P = torch.randn(2, B, W, device=dev).to(torch.bfloat16), torch.empty(2, B * top, 2 * ff, device=dev)
+    ahl, P2 = torch.randn(2, B * top, ff, device=dev).to(torch.bfloat16), torch.empty(2, B * top, W, device=dev)
+    t = _time_graph(lambda: lib().mn_stream_mfma_grouped(ptr(hilo), B, L.w_gate_up, 2 * ff * W, ptr(P), B * top, ptr(offsets), ptr(perm), E, B, 2 * ff, W,
+                                                         current_stream()))
+    record("expert_gate_up_decode_b32", t, byts=E * 2 * ff * W * 2)
+    t = _time_graph(lambda: lib().mn_stream_mfma_grouped(ptr(ahl), B * top, L.w_down, W * ff, ptr(P2), B * top, ptr(offsets), None, E, B, W, ff,
+                                                         current_stream()))
+    record("expert_down_decode_b32", t, byts=E * ff * W * 2)
+    t = _time_graph(lambda: check(lib().mn_gemm256_grouped_tiles_scaled(
+        ptr(h16), W, 0, B, ptr(perm), L.w_gate_up, W, 2 * ff * W, ptr(offsets), ptr(counts), E, ptr(tg), ptr(tm), ptr(nt), B * top // 256 + E, None,
+        ptr(act16), ff, 0, ff, W, 6, current_stream()), "mn_gemm256_grouped_tiles_scaled"))
+    record("tiles_gate_up_decode_b32", t, byts=E * 2 * ff * W * 2)
+    return out
+
+
+def run_sabezen_attention(s, T, batches, n_dec):
+    from .sabezen import SabezenDecoder
+    cfg = sabezen_config(s, dense=False, attention_only=True)
+    return _rates(SabezenDecoder.synthetic(cfg, "cuda", t_max=T + n_dec + 8, n_seq=max(batches), arith="bf16"), s, T, batches, n_dec)
+
+
 def run_bailing(s, T, batches, n_dec, shared=0):
     from . import ops
     from ._lib import check, current_stream, lib, ptr
@@ -614,6 +744,15 @@ def compare(sizes=("w1024", "w2048"), prompt=2048, batches=(1, 32), n_dec=32, mo
                              ("zuzenex_dense", lambda: run_zuzenex(s, prompt, batches, n_dec, dense=True)),
                              ("sabezen_moe", lambda: run_sabezen(s, prompt, batches, n_dec, dense=False, kernels=False)),
                              ("zuzenex_moe", lambda: run_zuzenex(s, prompt, batches, n_dec)), ("daberax", lambda: run_daberax(s, prompt, batches, n_dec))):
+                res[name][key] = run()
+                torch.cuda.empty_cache()
+                print(f"[lm-compare] {name} {key}", file=sys.stderr, flush=True)
+            continue
+        if model == "fegarax":                               # beside attention-only stacks of the models with the like kernels
+            res[name] = dict(size=s, prompt=prompt)
+            for key, run in (("fegarax", lambda: run_fegarax(s, prompt, batches, n_dec)),
+                             ("zuzenex_attention", lambda: run_zuzenex(s, prompt, batches, n_dec, attention_only=True)),
+                             ("sabezen_attention", lambda: run_sabezen_attention(s, prompt, batches, n_dec))):
                 res[name][key] = run()
                 torch.cuda.empty_cache()
                 print(f"[lm-compare] {name} {key}", file=sys.stderr, flush=True)

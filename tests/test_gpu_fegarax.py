@@ -188,6 +188,50 @@ def test_streams_update_combine_and_norm():
                     assert err(h, O.norm_zero(u, w, 1e-3)) < 5e-6 and bool((keep == dst).all())
 
 
+def test_streams_update_takes_the_router_along():
+    """The update also computes the router on the normed rows (fp32), picks and scores; few rows: expert results that lie in slabs, bf16 rows
+    with their low parts; every number of streams the form has, routers of 1 .. 300 outputs, rows of 8 .. 8192 values."""
+    from ming_univision_amd._lib import StreamsArgs
+    check, stream, L, ptr = _api()
+    g = torch.Generator().manual_seed(4)
+    for M, n, S, E, picks, top in ((1, 8, 1, 1, 1, 0), (5, 64, 3, 7, 3, 2), (64, 200, 2, 16, 2, 1), (3, 2048, 4, 8, 2, 2), (2, 8192, 4, 20, 5, 0), (7, 4104, 3, 65, 9, 3),
+                                   (20, 520, 1, 300, 4, 2), (2, 6000, 2, 33, 33, 1), (65, 64, 3, 16, 2, 2),
+                                   (100, 2056, 4, 8, 8, 1), (70, 8192, 2, 1, 1, 0), (90, 1000, 1, 5, 2, 3)):
+        few = M <= 64
+        X, y, slabs = torch.randn(M, S, n, generator=g), torch.randn(M, n, generator=g), 1 + (M % 3 if few else 0)
+        Z = max(1, M * top)
+        ye, slot, ew = torch.randn(slabs, Z, n, generator=g), torch.randperm(Z, generator=g).to(torch.int32), torch.rand(Z, generator=g)
+        mix, wi, wo = torch.randn(S, S, generator=g) * 0.5, torch.randn(S, generator=g), torch.randn(S, generator=g)
+        w, rt = _bf(0.2 * torch.randn(n, generator=g)), _bf(torch.randn(E, n, generator=g) * 3 * n ** -0.5)
+        assert L.mn_streams_router_ok(M, S, n, E, ptr(D(rt))) == 1
+        r = y.double()
+        for j in range(top):
+            z = torch.arange(M) * top + j
+            r = r + ew[z].double()[:, None] * ye.double().sum(0)[slot[z].long()]
+        new = O.streams_write(X.double().transpose(0, 1), r, mix, wo)
+        href = O.norm_zero(O.streams_read(new, wi), w, 1e-3)
+        zref = href @ rt.double().T
+        for both in (True, False):
+            dst, h, hl = X.clone().cuda(), torch.zeros(M, n, device="cuda"), torch.zeros(2, M, n, dtype=torch.bfloat16, device="cuda")
+            idx, pw = torch.full((M, picks), -1, dtype=torch.int32, device="cuda"), torch.zeros(M, picks, device="cuda")
+            a = StreamsArgs(src=dst.data_ptr(), src_row=S * n, src_stream=n, dst=dst.data_ptr(), S=S, n=n, mix=D(mix).data_ptr(), out=D(wo).data_ptr(),
+                            in_=D(wi).data_ptr(), y=D(y).data_ptr(), ldy=n, ye=D(ye).data_ptr(), ldye=n, slot_of=D(slot).data_ptr(), ew=D(ew).data_ptr(),
+                            top=top, one_plus=1, w=D(w).data_ptr(), eps=1e-3, h=h.data_ptr() if both else None, ldh=n, h16=hl.data_ptr(), ldh16=n,
+                            h16_lo=hl[1].data_ptr() if few else None, ye_slab=Z * n, ye_slabs=slabs, experts=E, router=D(rt).data_ptr(), idx=idx.data_ptr(), pw=pw.data_ptr(),
+                            picks=picks)
+            streams_call(a, M)
+            assert err(dst.transpose(0, 1), new) < 2e-6 and err(hl.double().sum(0), href) < (2e-5 if few else 1e-2), (M, n, S)
+            if both:
+                assert err(h, href) < 5e-6
+            got = torch.gather(zref, 1, idx.cpu().long())            # the picks: distinct, in falling order, the largest up to rounding
+            assert all(len(set(row)) == picks for row in idx.tolist())
+            assert float((got - torch.topk(zref, picks, dim=1).values).abs().max()) < 2e-5 * float(zref.abs().max())
+            assert float((pw.double().cpu() - torch.sigmoid(got)).abs().max()) < 2e-5
+    t = D(torch.zeros(4, 64, dtype=torch.bfloat16))
+    assert L.mn_streams_router_ok(65, 3, 64, 17, ptr(t)) == 0 and L.mn_streams_router_ok(64, 3, 64, 513, ptr(t)) == 0 and L.mn_streams_router_ok(5, 5, 64, 4, ptr(t)) == 0
+    assert L.mn_streams_router_ok(5, 3, 60, 4, ptr(t)) == 0 and L.mn_streams_router_ok(5, 3, 8200, 4, ptr(t)) == 0
+
+
 def test_streams_refuse_what_they_do_not_take():
     from ming_univision_amd._lib import StreamsArgs
     t = torch.zeros(2, 33, 8, device="cuda")
@@ -339,7 +383,8 @@ def glu(x, w, s):
 
 
 def test_experts_are_fed_with_weight_times_input():
-    """The three routes: pair by pair, the grouped product followed by the activation, the 256-tile product with its scaled epilogue."""
+    """The routes: pair by pair, the grouped product followed by the activation, the 256-tile product with its scaled epilogue, the grouped
+    weight-streaming product (few rows, high and low bf16 parts: fp32-class results)."""
     check, stream, L, ptr = _api()
     g = torch.Generator().manual_seed(3)
     for M, top, E, N, K in ((3, 2, 5, 24, 64), (4, 3, 4, 14, 44), (1, 1, 1, 8, 2048), (8, 2, 8, 100, 520), (90, 2, 6, 64, 128), (300, 3, 4, 192, 64), (40, 1, 3, 40, 72)):
@@ -380,6 +425,14 @@ def test_experts_are_fed_with_weight_times_input():
                 assert err(y32, O.silu(gu[:, :N].double().cpu()) * gu[:, N:].double().cpu()) < 1e-6
                 _KEEP.append((xg, gu))
             assert err(y16.float()[slot.long()], ref) < 2e-2, (M, N, K, tiles)
+        if M <= 64 and int(counts.max()) <= 64:
+            hi = _bf(x)
+            Y = D(torch.stack([hi, _bf(x - hi.float())]).contiguous())
+            P, y2 = torch.zeros(2, Z, 2 * N, device="cuda"), torch.zeros(2, Z, N, dtype=torch.bfloat16, device="cuda")
+            nz = L.mn_stream_mfma_grouped(ptr(Y), M, ptr(wd), 2 * N * K, ptr(P), Z, ptr(offsets), ptr(perm), E, min(64, Z), 2 * N, K, stream())
+            assert 1 <= nz <= 2
+            check(L.mn_silu_split_rows_scaled(ptr(P), nz, Z, N, ptr(ws), ptr(y2), stream()))
+            assert err(y2.double().sum(0)[slot.long()], ref) < 1e-4, (M, N, K)
 
 
 # ---- whole models ------------------------------------------------------------------------------------------------------------
