@@ -263,6 +263,15 @@ extern "C" int mn_moe_router(const float* x, int64_t ldx, const uint16_t* norm_w
   return MN_OK;
 }
 
+// One rotary pair.  The products are rounded before they are added (no contraction), like the rotation they stand for: what a fused form
+// would round once less depends on which of the two products the compiler folds in.
+__device__ __forceinline__ void rotate_pair(float& x1, float& x2, float c, float s) {
+#pragma clang fp contract(off)
+  const float a = x1 * c, b = x2 * s, d = x2 * c, e = x1 * s;
+  x1 = a - b;
+  x2 = d + e;
+}
+
 // -------------------------------------------------------------------------------------------
 // RoPE + KV append. grid (M, n_q + 2*n_kv), block hd/2 threads.
 // -------------------------------------------------------------------------------------------
@@ -293,8 +302,7 @@ __global__ void rope_kv_append_kernel(const float* __restrict__ qkv, int64_t ldq
     const int stream = sec_t <= 0 ? 0 : (i < sec_t ? 0 : (i < sec_t + sec_h ? 1 : 2));
     const int pos = row_pos[stream * M + m];
     const float c = cos_tab[(int64_t)pos * half + i], s = sin_tab[(int64_t)pos * half + i];
-    const float o1 = x1 * c - x2 * s, o2 = x2 * c + x1 * s;
-    x1 = o1; x2 = o2;
+    rotate_pair(x1, x2, c, s);
   }
   if (is_q) {
     float* dst = q_out + (int64_t)m * n_q * hd + (int64_t)h * hd;
@@ -732,8 +740,7 @@ __global__ __launch_bounds__(1024) void attn_decode_one_kernel(
         const int stream = fz.sec_t <= 0 ? 0 : (lane < fz.sec_t ? 0 : (lane < fz.sec_t + fz.sec_h ? 1 : 2));
         const int pos = fz.row_pos[stream * fz.M + m];
         const float c = fz.cos_tab[(int64_t)pos * half + lane], sn = fz.sin_tab[(int64_t)pos * half + lane];
-        const float o1 = x1 * c - x2 * sn, o2 = x2 * c + x1 * sn;
-        x1 = o1; x2 = o2;
+        rotate_pair(x1, x2, c, sn);
       }
       if (wave == 0) { x1 *= fz.q_scale; x2 *= fz.q_scale; }
       float* dst = wave == 0 ? qs : (wave == 1 ? knew : vnew);
